@@ -633,7 +633,11 @@ constexpr int kMaxDevices = 64;
 static __device__ __align__(256) unsigned char scratch[kStaticScratchBytes];
 static void* g_scratch_ptr[kMaxDevices] = {};
 
-namespace dh {
+namespace {
+using dh::Graph;
+using dh::GraphAttnCall;
+using dh::fail;
+
 // The captured graph is a chain (one stream): walking it from its root visits the kernel nodes in
 // launch order.  Every recorded attention call owns the next node that runs its split kernel and
 // the merge node behind it.
@@ -738,6 +742,8 @@ int attn_graph_set_position(Graph* g, int position) {
   return 0;
 }
 
+// Looks up, once per device, the address of the fixed device array that dh_attn_decode_static uses for its
+// split partials.  Called by dh_init with the device current.
 int attn_static_scratch_init(int device) {
   if (device < 0 || device >= kMaxDevices)
     return fail(1, "[dh_init] device ordinal %d is beyond the %d the static attention scratch tracks", device, kMaxDevices);
@@ -747,7 +753,9 @@ int attn_static_scratch_init(int device) {
   g_scratch_ptr[device] = ptr;
   return 0;
 }
-}  // namespace dh
+
+const int g_family = dh::register_family({attn_static_scratch_init, nullptr, nullptr, attn_graph_bind, attn_graph_set_position});
+}  // namespace
 
 
 extern "C" {

@@ -79,12 +79,20 @@ const int64_t* plan_layout_record();
 uint32_t* kernel_status_word();
 // Reads and clears the word (call only after the stream has been synchronised); non-zero -> fail().
 int check_kernel_status(const char* op);
-// chained GEMV (q4k_gemv_chain.hip): called when a launch has reported a failed wait, so that the
-// next launch starts from a clean exchange area.
-void gemv_chain_reset();
-// chained GEMV: exchange area and launch counter (allocated by dh_init, freed with the runtime).
-int gemv_chain_init(int device);
-void gemv_chain_release();
+
+// ---- kernel families with state of their own --------------------------------------------------
+// What the runtime calls on a family's behalf; a null entry is skipped.  A family registers itself when
+// the library is loaded, so the runtime names none of them and a library may be linked from the families
+// one kind of model needs.
+struct Graph;
+struct Family {
+  int (*init)(int device);                              // dh_init, device current
+  void (*release)();                                    // the runtime is being released
+  void (*reset)();                                      // a launch reported a failed wait: start clean
+  int (*graph_bind)(Graph* g);                          // a capture has ended
+  int (*graph_set_position)(Graph* g, int position);    // a captured step moves to another position
+};
+int register_family(const Family& f);
 
 // Matrix-core GEMM for prefill-sized batches (q4k_gemm.hip).  `serves`: M >= 16, K a multiple
 // of 4, A 16-byte aligned.
@@ -148,18 +156,11 @@ struct Graph {
 Graph* capturing_graph();
 // attention.hip: records a call for the graph being captured (no-op outside a capture).
 void graph_note_attention(const GraphAttnCall& call);
-// attention.hip: finds the kernel nodes of the recorded calls in the captured graph / patches them for `position`.
-int attn_graph_bind(Graph* g);
-int attn_graph_set_position(Graph* g, int position);
 // elementwise.hip: the same for the finiteness checks of a captured step (their step number is a
 // launch argument: a replay at position p reports captured step + p - captured position).
 void graph_note_finiteness(const GraphFiniteCall& call);
 int finite_graph_bind(Graph* g);
 int finite_graph_set_position(Graph* g, int position);
-
-// Looks up, once per device, the address of the fixed device array that dh_attn_decode_static uses
-// for its split partials (attention.hip).  Called by dh_init with the device current.
-int attn_static_scratch_init(int device);
 
 // Decode GEMV on the int8 matrix cores (q4k_gemv_i8.hip): C = alpha * A . W^T + residual, or with W2
 // the gated pair act(A . W^T) * (A . W2^T) * alpha; norm_weight != null normalises A's rows first.

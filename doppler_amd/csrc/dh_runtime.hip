@@ -12,6 +12,9 @@ int g_device = -1;
 hipStream_t g_own_stream = nullptr;
 hipStream_t g_stream = nullptr;
 int g_num_cus = 0;
+constexpr int kMaxFamilies = 16;
+dh::Family g_families[kMaxFamilies];  // filled while the library is being loaded (zero-initialised before that)
+int g_num_families;
 dh::Graph* g_capturing = nullptr;     // graph being captured on g_stream
 float* g_splitk_ws = nullptr;        // partial products of the split-K prefill GEMM
 constexpr size_t kSplitKWsBytes = (size_t)32 << 20;
@@ -34,6 +37,11 @@ int fail(int code, const char* fmt, ...) {
   vsnprintf(g_err, sizeof(g_err), fmt, ap);
   va_end(ap);
   return code;
+}
+int register_family(const Family& f) {
+  if (g_num_families >= kMaxFamilies) abort();
+  g_families[g_num_families] = f;
+  return g_num_families++;
 }
 hipStream_t stream() { return g_stream; }
 bool ready() { return g_ready || t_plan_cus > 0; }
@@ -104,7 +112,8 @@ int check_kernel_status(const char* op) {
   const uint32_t code = *static_cast<volatile uint32_t*>(g_kstatus);
   if (code == 0u) return 0;
   *static_cast<volatile uint32_t*>(g_kstatus) = 0u;
-  gemv_chain_reset();
+  for (int i = 0; i < g_num_families; i++)
+    if (g_families[i].reset) g_families[i].reset();
   const uint32_t kind = code >> 28, phase = (code >> 24) & 0xFu, block = code & 0xFFFFFFu;
   const char* what = kind == DH_KSTATUS_COLUMN_WAIT ? "a column's activation operands did not arrive (Q4_K GEMV)"
                      : kind == DH_KSTATUS_SLOT_WAIT ? "a tile slot was not released (Q4_K GEMV)"
@@ -142,7 +151,8 @@ static int release_all(const char* op) {
   if (g_packed_a) note(hipFree(g_packed_a));
   if (g_widened_a) note(hipFree(g_widened_a));
   if (g_kstatus) note(hipHostFree(g_kstatus));
-  dh::gemv_chain_release();
+  for (int i = 0; i < g_num_families; i++)
+    if (g_families[i].release) g_families[i].release();
   g_own_stream = nullptr;
   g_stream = nullptr;
   g_splitk_ws = nullptr;
@@ -177,8 +187,10 @@ static int init_locked(int device_ordinal) {
   DH_CHECK_HIP("dh_init", hipMalloc(reinterpret_cast<void**>(&g_widened_a), kWidenedABytes));
   DH_CHECK_HIP("dh_init", hipHostMalloc(reinterpret_cast<void**>(&g_kstatus), 64, hipHostMallocMapped));
   *g_kstatus = 0u;
-  if (int rc = dh::attn_static_scratch_init(device_ordinal)) return rc;
-  if (int rc = dh::gemv_chain_init(device_ordinal)) return rc;
+  for (int i = 0; i < g_num_families; i++) {
+    if (!g_families[i].init) continue;
+    if (int rc = g_families[i].init(device_ordinal)) return rc;
+  }
   g_device = device_ordinal;
   g_ready = true;
   return 0;
@@ -368,6 +380,16 @@ int dh_graph_begin(void) {
   return 0;
 }
 
+static int graph_move(dh::Graph* g, int position) {
+  for (int i = 0; i < g_num_families; i++) {
+    if (!g_families[i].graph_set_position) continue;
+    if (int rc = g_families[i].graph_set_position(g, position)) return rc;
+  }
+  if (int rc = dh::finite_graph_set_position(g, position)) return rc;
+  g->position = position;
+  return 0;
+}
+
 static void graph_free(dh::Graph* g) {
   if (!g) return;
   if (g->exec) (void)hipGraphExecDestroy(g->exec);
@@ -395,9 +417,12 @@ int dh_graph_end(int position, void** graph_out) {
     return dh::fail(2, "[dh_graph_end] hipGraphInstantiate failed: %s", hipGetErrorString(e));
   }
   g->position = g->captured_position = position;
-  if (int rc = dh::attn_graph_bind(g)) {
-    graph_free(g);
-    return rc;
+  for (int i = 0; i < g_num_families; i++) {
+    if (!g_families[i].graph_bind) continue;
+    if (int rc = g_families[i].graph_bind(g)) {
+      graph_free(g);
+      return rc;
+    }
   }
   if (int rc = dh::finite_graph_bind(g)) {
     graph_free(g);
@@ -427,9 +452,7 @@ int dh_graph_launch(void* graph, int position) {
     return dh::fail(1, "[dh_graph_launch] position %d is beyond the largest one the step's buffers were declared for (%d)",
                     position, g->max_position);
   if (position != g->position) {
-    if (int rc = dh::attn_graph_set_position(g, position)) return rc;
-    if (int rc = dh::finite_graph_set_position(g, position)) return rc;
-    g->position = position;
+    if (int rc = graph_move(g, position)) return rc;
   }
   DH_CHECK_HIP("dh_graph_launch", hipGraphLaunch(g->exec, g_stream));
   return 0;
@@ -445,9 +468,7 @@ int dh_graph_prepare(void* graph, int position) {
     return dh::fail(1, "[dh_graph_prepare] position %d is beyond the largest one the step's buffers were declared for (%d)",
                     position, g->max_position);
   if (position != g->position) {
-    if (int rc = dh::attn_graph_set_position(g, position)) return rc;
-    if (int rc = dh::finite_graph_set_position(g, position)) return rc;
-    g->position = position;
+    if (int rc = graph_move(g, position)) return rc;
   }
   return 0;
 }

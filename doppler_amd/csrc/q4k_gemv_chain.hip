@@ -883,10 +883,7 @@ int launch(const char* op, Plan& plan, int workgroups) {
   return 0;
 }
 
-}  // namespace
-
-namespace dh {
-
+// Exchange area and launch counter.
 int gemv_chain_init(int) {
   DH_CHECK_HIP("dh_init", hipMalloc(reinterpret_cast<void**>(&g_ll), (size_t)2 * kMaxChainN * sizeof(v2u)));
   DH_CHECK_HIP("dh_init", hipMalloc(reinterpret_cast<void**>(&g_epoch), 256));
@@ -914,7 +911,9 @@ void gemv_chain_reset() {
   (void)hipMemcpy(g_epoch, &e, 4, hipMemcpyHostToDevice);
 }
 
-}  // namespace dh
+const int g_family = dh::register_family({gemv_chain_init, gemv_chain_release, gemv_chain_reset, nullptr, nullptr});
+
+}  // namespace
 
 extern "C" {
 
