@@ -3,6 +3,7 @@ Node-API addon that binds it for the JavaScript host code.
 
     python -m doppler_amd.build            # everything
     python -m doppler_amd.build --hip-only
+    python -m doppler_amd.build --dense    # only what dense-weight models run on
 
 hipcc cross-compiles for gfx950 without a GPU present.  The flag pair
 `-Xclang -target-feature -Xclang -packed-fp32-ops` keeps the compiler from forming packed
@@ -41,16 +42,28 @@ def _run(cmd):
         print(out)
 
 
-def build_hip(jobs=4):
+# The families a model with dense weights runs on: the runtime, its glue ops, output heads and sampling, the dense
+# products and the attention they feed.
+DENSE_SOURCES = ("attention_prefill.hip", "attention_spec.hip", "dense_elementwise.hip", "dense_gemm.hip", "dense_gemv.hip",
+                 "dh_runtime.hip", "elementwise.hip", "lmhead.hip", "sample.hip")
+DENSE_LIB = os.path.join(LIB_DIR, "libdopplerhip_dense.so")
+
+
+def build_dense(jobs=8):
+    """Compiles the dense families alone and links them into a library of their own; returns its path."""
+    return build_hip(jobs, [os.path.join(CSRC, s) for s in DENSE_SOURCES], DENSE_LIB)
+
+
+def build_hip(jobs=4, srcs=None, lib=LIB):
     os.makedirs(OBJ, exist_ok=True)
     os.makedirs(LIB_DIR, exist_ok=True)
-    srcs = sorted(glob.glob(os.path.join(CSRC, "*.hip")))
+    srcs = srcs or sorted(glob.glob(os.path.join(CSRC, "*.hip")))
     objs = [os.path.join(OBJ, os.path.basename(s)[:-4] + ".o") for s in srcs]
     with ThreadPoolExecutor(max_workers=jobs) as ex:
         list(ex.map(lambda so: _run([HIPCC] + HIP_FLAGS + FILE_FLAGS.get(os.path.basename(so[0]), []) +
                                     ["-c", so[0], "-o", so[1]]), zip(srcs, objs)))
-    _run([HIPCC, "--offload-arch=gfx950", "-shared", "-fPIC", "-o", LIB] + objs)
-    return LIB
+    _run([HIPCC, "--offload-arch=gfx950", "-shared", "-fPIC", "-o", lib] + objs)
+    return lib
 
 
 def build_addon():
@@ -75,6 +88,7 @@ def build_all(hip_only=False):
 if __name__ == "__main__":
     ap = argparse.ArgumentParser()
     ap.add_argument("--hip-only", action="store_true")
+    ap.add_argument("--dense", action="store_true")
     args = ap.parse_args()
-    print(build_all(args.hip_only))
+    print(build_dense() if args.dense else build_all(args.hip_only))
     sys.exit(0)

@@ -8,9 +8,11 @@ import os
 
 _HERE = os.path.dirname(os.path.abspath(__file__))
 LIB_PATH = os.path.join(_HERE, "lib", "libdopplerhip.so")
+# the library linked from the kernel families dense-weight models need (doppler_amd.build.build_dense)
+DENSE_LIB_PATH = os.path.join(_HERE, "lib", "libdopplerhip_dense.so")
 
-F32, F16 = 0, 1
-ACT_SILU, ACT_GELU = 0, 1
+F32, F16, BF16 = 0, 1, 2
+ACT_SILU, ACT_GELU, ACT_RELU2, ACT_NONE = 0, 1, 2, -1
 KV_CONTIGUOUS, KV_RING = 0, 1
 PLAN_GEMV_I8, PLAN_GEMV_ROWS, PLAN_GEMV_RING, PLAN_GEMM, PLAN_GEMV_LDS = 1, 2, 3, 4, 5
 
@@ -36,6 +38,13 @@ class ChainAttnSource(ctypes.Structure):
     """struct dh_chain_attn_source: the attention partial results a chain's first product merges."""
     _fields_ = [("d_workspace", _P), ("H", _I), ("Hkv", _I), ("D", _I), ("nsplit", _I), ("d_kv_len", _P),
                 ("max_kv_len", _I), ("sliding_window", _I), ("kv_start", _I)]
+
+
+class AttnSpec(ctypes.Structure):
+    """struct dh_attn_spec: one layer's attention with distance bias, window, value norm and output gate."""
+    _fields_ = [("H", _I), ("Hkv", _I), ("D", _I), ("VD", _I), ("value_dim", _I), ("window", _I), ("cache_dtype", _I),
+                ("value_norm", _I), ("k_offset", _I), ("v_offset", _I), ("gate_offset", _I), ("ld_qkv", _I),
+                ("scale", _F), ("value_eps", _F), ("d_bias_r1", _P), ("d_bias_r2", _P)]
 
 
 def chain_phases(phases):
@@ -107,6 +116,15 @@ SIGNATURES = {
                                          _I, _P, ctypes.POINTER(_I)]),
     "dh_attn_decode_qkv_kvlen_partials": (_I, [_P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _P, _I, _I, _I, _F, _I, _I, _F, _F,
                                                _I, _I, _I, _P]),
+    "dh_dense_matmul": (_I, [_P, _I, _I, _P, _I, _I, _I, _I, _F, _P, _P, _P, _I, _I, _P, _I, _I, _I]),
+    "dh_dense_gemv": (_I, [_P, _P, _I, _F, _P, _I, _I, _I, _F, _P, _P, _P, _I, _P, _I]),
+    "dh_dense_lmhead_argmax": (_I, [_P, _P, _I, _F, _P, _I, _I, _I, _F, _P, _P, _I, _P]),
+    "dh_embed_sum": (_I, [_P, _I, _P, _P, _I, _P, _I64, _I64, _I64, _P, _I, _P, _I, _I, _I, _I, _P]),
+    "dh_rmsnorm_rows": (_I, [_P, _I, _P, _P, _P, _I, _I, _I, _I, _F]),
+    "dh_attn_spec_workspace_bytes": (_SZ, [_I, _I, _I]),
+    "dh_attn_spec_kv_write": (_I, [ctypes.POINTER(AttnSpec), _P, _P, _P, _I, _I]),
+    "dh_attn_spec_prefill": (_I, [ctypes.POINTER(AttnSpec), _P, _P, _P, _P, _I, _I, _I, _I]),
+    "dh_attn_spec_decode": (_I, [ctypes.POINTER(AttnSpec), _P, _P, _P, _P, _I, _P, _I, _P]),
     "dh_rmsnorm": (_I, [_P, _P, _I, _P, _I, _I, _F, _I, _P, _P, _P, _F]),
     "dh_rmsnorm_sandwich_pair": (_I, [_P, _P, _P, _I, _P, _I, _P, _P, _I, _I, _F, _I]),
     "dh_residual_rmsnorm_pair": (_I, [_P, _P, _P, _I, _P, _P, _I, _I, _F, _I, _F]),
@@ -139,15 +157,21 @@ SIGNATURES = {
 _lib = None
 
 
-def load():
-    """Loads the shared library (no GPU needed for loading) and types every symbol."""
+def load(path=None):
+    """Loads the shared library (no GPU needed for loading) and types every symbol.  path: another library to bind
+    instead of the whole one, before anything else has loaded it; it may lack families (calling an op it lacks
+    fails)."""
     global _lib
     if _lib is None:
-        if not os.path.exists(LIB_PATH):
+        partial = path is not None
+        path = path or LIB_PATH
+        if not os.path.exists(path):
             raise DopplerHipError(
-                "libdopplerhip.so is not built (expected %s); run `python -m doppler_amd.build`" % LIB_PATH)
-        lib = ctypes.CDLL(LIB_PATH)
+                "libdopplerhip.so is not built (expected %s); run `python -m doppler_amd.build`" % path)
+        lib = ctypes.CDLL(path)
         for name, (res, args) in SIGNATURES.items():
+            if partial and not hasattr(lib, name):
+                continue
             fn = getattr(lib, name)
             fn.restype = res
             fn.argtypes = args

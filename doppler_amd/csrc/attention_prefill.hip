@@ -22,13 +22,19 @@
 //                   renumbered as long as both operands agree), A = V^T read from LDS, where the
 //                   V tile was stored transposed with its keys in that same slot order.
 // Causal tiles beyond the tile's last query are never visited.
+// The SPEC form (dh_attn_spec_prefill) serves the attention of decoders without rotary positions: queries are read
+// from stacked projection rows, every score loses r1 log2(1 + r2 (i - j)) (the distance bias in the softmax's own
+// units), value heads may differ in size from key heads (both are padded to the template's sizes with zeros in
+// LDS and registers), probabilities enter the second product as f16 high part + residual (22 bits), and the output is
+// gated per head and written in the operand type of the product that reads it.
 // (Measured without effect at T = 2048..4096: a second LDS buffer per tile with one barrier per
 // tile instead of two, and dispatching the long late-query tiles first.)
 #include <algorithm>
 #include <cfloat>
 #include <cstdlib>
 
-#include "dh_common.h"
+#include "attention_spec.h"
+#include "dense_device.h"
 
 namespace {
 
@@ -62,26 +68,35 @@ struct PrefillArgs {
   float* O;             // [T][H][D]
   int T, H, Hkv, G, kv_len, start_pos, causal, window;
   float scale, softcap;
+  // ---- SPEC form only
+  int dk, dv;           // head sizes of caches and projection rows (<= the template's, multiples of 8)
+  int64_t ld_q, ld_o;
+  const float* r1;      // [H] or null
+  const float* r2;
+  const float* gate;    // H numbers per query token, ld_q apart, or null
+  uint16_t* O16;        // bf16 output instead of O
 };
 
 // QT = 16-query groups per wave: every K and V fragment read from LDS feeds QT matrix-core
 // instructions, and a workgroup tile (64 QT queries) stages each key tile once.
-template <int D, int QT>
+template <int D, int VD, int QT, bool SPEC>
 __global__ __launch_bounds__(256) void attn_prefill_kernel(const PrefillArgs a) {
   constexpr int BQ = 64 * QT;
   constexpr int STEPS = D / 32;            // MFMAs per 16 x 16 score tile
-  constexpr int DT = D / 16;               // output row tiles (of O^T)
+  constexpr int DT = VD / 16;              // output row tiles (of O^T)
   constexpr int KROW = D + 8;              // halves per K row in LDS (16-byte pad)
   constexpr int VROW = BKEYS + 8;          // halves per V^T row in LDS
-  constexpr int PIECES = BKEYS * D / 8 / 256;   // 16-byte pieces of a tile per thread
+  constexpr int PIECES = BKEYS * D / 8 / 256;   // 16-byte pieces of a K tile per thread
+  constexpr int VPIECES = BKEYS * VD / 8 / 256;
   __shared__ __align__(16) _Float16 k_lds[BKEYS * KROW];
-  __shared__ __align__(16) _Float16 v_lds[D * VROW];
+  __shared__ __align__(16) _Float16 v_lds[VD * VROW];
 
   const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63;
   const int q = lane & 15, g = lane >> 4;
   const int h = blockIdx.y, kvh = h / a.G;
   const int q0 = blockIdx.x * BQ;
-  const int64_t kv_stride = (int64_t)a.Hkv * D;
+  const int dk = SPEC ? a.dk : D, dv = SPEC ? a.dv : VD;
+  const int64_t k_stride = (int64_t)a.Hkv * dk, v_stride = (int64_t)a.Hkv * dv;
   int my_q[QT], my_pos[QT];                                   // query token of this lane's column, its absolute position
 #pragma unroll
   for (int u = 0; u < QT; u++) {
@@ -99,8 +114,10 @@ __global__ __launch_bounds__(256) void attn_prefill_kernel(const PrefillArgs a) 
   for (int u = 0; u < QT; u++)
 #pragma unroll
     for (int s = 0; s < STEPS; s++) {
-      const float* qp = a.Q + ((int64_t)min(my_q[u], a.T - 1) * a.H + h) * D + 32 * s + 8 * g;
-      const float4 v0 = reinterpret_cast<const float4*>(qp)[0], v1 = reinterpret_cast<const float4*>(qp)[1];
+      const int64_t qrow = min(my_q[u], a.T - 1);
+      const float* qp = a.Q + (SPEC ? qrow * a.ld_q + (int64_t)h * dk : (qrow * a.H + h) * D) + 32 * s + 8 * g;
+      float4 v0 = make_float4(0.f, 0.f, 0.f, 0.f), v1 = v0;
+      if (!SPEC || 32 * s + 8 * g < dk) { v0 = reinterpret_cast<const float4*>(qp)[0]; v1 = reinterpret_cast<const float4*>(qp)[1]; }
       const float qv[8] = {v0.x, v0.y, v0.z, v0.w, v1.x, v1.y, v1.z, v1.w};
 #pragma unroll
       for (int i = 0; i < 8; i++) qb[u][s][i] = (_Float16)(qv[i] * qscale);
@@ -115,6 +132,11 @@ __global__ __launch_bounds__(256) void attn_prefill_kernel(const PrefillArgs a) 
   kbeg = kbeg / BKEYS * BKEYS;
   const int ntiles = (kend - kbeg + BKEYS - 1) / BKEYS;
 
+  float r1 = 0.f, r2 = 0.f;
+  if (SPEC && a.r1) {
+    r1 = a.r1[h];
+    r2 = a.r2[h];
+  }
   float4_t acc[QT][DT];
   float m_run[QT], l_run[QT];
 #pragma unroll
@@ -125,7 +147,7 @@ __global__ __launch_bounds__(256) void attn_prefill_kernel(const PrefillArgs a) 
     l_run[u] = 0.f;
   }
 
-  u32x4_t kreg[PIECES], vreg[PIECES];
+  u32x4_t kreg[PIECES], vreg[VPIECES];
   // K piece p = tid + 256 r of a tile: key p / (D/8), 8 consecutive dims starting at 8 (p % (D/8)).
   // V is fetched by key PAIRS, so that the transposed tile can be written in 32-bit words: item j
   // of a thread is keys 2 (tid % 32), 2 (tid % 32) + 1 and dims 8 c .. 8 c + 7, c = tid / 32 + 8 j
@@ -136,10 +158,16 @@ __global__ __launch_bounds__(256) void attn_prefill_kernel(const PrefillArgs a) 
   _Pragma("unroll") for (int r = 0; r < PIECES; r++) {                                           \
     const int p_ = tid + 256 * r, key_ = p_ / (D / 8), c_ = p_ % (D / 8);                        \
     const int row_ = min(kbeg + (tile_) * BKEYS + key_, a.kv_len - 1);                           \
-    kreg[r] = *reinterpret_cast<const u32x4_t*>(a.K + (int64_t)row_ * kv_stride + (int64_t)kvh * D + 8 * c_); \
+    kreg[r] = u32x4_t{0u, 0u, 0u, 0u};                                                           \
+    if (!SPEC || 8 * c_ < dk)                                                                    \
+      kreg[r] = *reinterpret_cast<const u32x4_t*>(a.K + (int64_t)row_ * k_stride + (int64_t)kvh * dk + 8 * c_); \
+  }                                                                                              \
+  _Pragma("unroll") for (int r = 0; r < VPIECES; r++) {                                          \
     const int vrow_ = min(kbeg + (tile_) * BKEYS + 2 * vpair + (r & 1), a.kv_len - 1);           \
-    vreg[r] = *reinterpret_cast<const u32x4_t*>(a.V + (int64_t)vrow_ * kv_stride + (int64_t)kvh * D + \
-                                              8 * (vcol + 8 * (r >> 1)));                        \
+    const int c_ = vcol + 8 * (r >> 1);                                                          \
+    vreg[r] = u32x4_t{0u, 0u, 0u, 0u};                                                           \
+    if (!SPEC || 8 * c_ < dv)                                                                    \
+      vreg[r] = *reinterpret_cast<const u32x4_t*>(a.V + (int64_t)vrow_ * v_stride + (int64_t)kvh * dv + 8 * c_); \
   }
   if (ntiles > 0) { DH_PF_LOAD(0); }
 
@@ -156,7 +184,7 @@ __global__ __launch_bounds__(256) void attn_prefill_kernel(const PrefillArgs a) 
       const int key0 = 2 * vpair;
       const int slot = 32 * (key0 >> 5) + 8 * ((key0 >> 2) & 3) + 4 * ((key0 >> 4) & 1) + (key0 & 3);
 #pragma unroll
-      for (int j = 0; j < PIECES / 2; j++) {
+      for (int j = 0; j < VPIECES / 2; j++) {
         const int c = vcol + 8 * j;
         const u32x4_t aw = vreg[2 * j];
         const u32x4_t bw = vreg[2 * j + 1];
@@ -187,6 +215,7 @@ __global__ __launch_bounds__(256) void attn_prefill_kernel(const PrefillArgs a) 
     // ---- mask, soft cap, online softmax (this lane: query my_q, keys kbase + 16 j + 4 g + i).
     // A tile that every query of a 16-query group sees completely needs no per-element masks.
     half8_t pb[QT][2];
+    half8_t pl[SPEC ? QT : 1][2];            // SPEC: what the f16 probabilities left over
     float alpha[QT];
     bool rescale = false;
 #pragma unroll
@@ -195,6 +224,14 @@ __global__ __launch_bounds__(256) void attn_prefill_kernel(const PrefillArgs a) 
       const bool full = kbase + BKEYS <= a.kv_len && (!a.causal || kbase + BKEYS - 1 <= grp_lo) &&
                         (a.window <= 0 || kbase > grp_hi - a.window);
       float mx = -FLT_MAX;
+      if (SPEC && a.r1) {
+        const float d0 = (float)(my_pos[u] - kbase - 4 * g);
+#pragma unroll
+        for (int j = 0; j < 4; j++)
+#pragma unroll
+          for (int i = 0; i < 4; i++)         // keys behind the query give NaN or less; they are masked below
+            st[u][j][i] = fmaf(-r1, __builtin_amdgcn_logf(fmaf(r2, d0 - (float)(16 * j + i), 1.0f)), st[u][j][i]);
+      }
       if (full && !(a.softcap > 0.f)) {
 #pragma unroll
         for (int j = 0; j < 4; j++)
@@ -226,7 +263,9 @@ __global__ __launch_bounds__(256) void attn_prefill_kernel(const PrefillArgs a) 
         for (int i = 0; i < 4; i++) {
           const float p = __builtin_amdgcn_exp2f(st[u][j][i] - m_new);   // 2^-inf = 0 for masked keys
           ps += p;
-          pb[u][j >> 1][4 * (j & 1) + i] = (_Float16)p;
+          const _Float16 ph = (_Float16)p;
+          pb[u][j >> 1][4 * (j & 1) + i] = ph;
+          if constexpr (SPEC) pl[u][j >> 1][4 * (j & 1) + i] = (_Float16)(p - (float)ph);
         }
       l_run[u] = l_run[u] * alpha[u] + ps;               // this lane's share: alpha is the query's, the sum is taken once at the end
       m_run[u] = m_new;
@@ -244,6 +283,10 @@ __global__ __launch_bounds__(256) void attn_prefill_kernel(const PrefillArgs a) 
         const half8_t va = *reinterpret_cast<const half8_t*>(&v_lds[(16 * t + q) * VROW + 32 * kb + 8 * g]);
 #pragma unroll
         for (int u = 0; u < QT; u++) acc[u][t] = __builtin_amdgcn_mfma_f32_16x16x32_f16(va, pb[u][kb], acc[u][t], 0, 0, 0);
+        if constexpr (SPEC) {
+#pragma unroll
+          for (int u = 0; u < QT; u++) acc[u][t] = __builtin_amdgcn_mfma_f32_16x16x32_f16(va, pl[u][kb], acc[u][t], 0, 0, 0);
+        }
       }
     }
   }
@@ -254,7 +297,25 @@ __global__ __launch_bounds__(256) void attn_prefill_kernel(const PrefillArgs a) 
   for (int u = 0; u < QT; u++) {
     const float l = quad_rows_sum(l_run[u]);
     if (my_q[u] < a.T) {
-      const float inv = l > 0.f ? 1.0f / l : 0.f;
+      float inv = l > 0.f ? 1.0f / l : 0.f;
+      if constexpr (SPEC) {
+        if (a.gate) inv *= 1.0f / (1.0f + expf(-a.gate[(int64_t)my_q[u] * a.ld_q + h]));
+        const int64_t at = (int64_t)my_q[u] * a.ld_o + (int64_t)h * dv + 4 * g;
+#pragma unroll
+        for (int t = 0; t < DT; t++) {
+          if (16 * t + 4 * g >= dv) continue;
+          if (a.O16) {
+            uint2 two;
+            two.x = (uint32_t)dh::f32_to_bf16_bits(acc[u][t][0] * inv) | ((uint32_t)dh::f32_to_bf16_bits(acc[u][t][1] * inv) << 16);
+            two.y = (uint32_t)dh::f32_to_bf16_bits(acc[u][t][2] * inv) | ((uint32_t)dh::f32_to_bf16_bits(acc[u][t][3] * inv) << 16);
+            *reinterpret_cast<uint2*>(a.O16 + at + 16 * t) = two;
+          } else {
+            *reinterpret_cast<float4*>(a.O + at + 16 * t) =
+                make_float4(acc[u][t][0] * inv, acc[u][t][1] * inv, acc[u][t][2] * inv, acc[u][t][3] * inv);
+          }
+        }
+        continue;
+      }
       float* op = a.O + ((int64_t)my_q[u] * a.H + h) * D + 4 * g;
 #pragma unroll
       for (int t = 0; t < DT; t++)
@@ -293,12 +354,51 @@ extern "C" int dh_attn_prefill(const float* d_Q, const void* d_K, const void* d_
   const int qt = env_qt ? env_qt : ((int64_t)dh::ceil_div(T, 128) * H >= 2 * dh::num_cus() ? 2 : 1);
   const dim3 grid((unsigned)dh::ceil_div(T, 64 * qt), (unsigned)H);
   if (D == 64) {
-    if (qt == 2) hipLaunchKernelGGL((attn_prefill_kernel<64, 2>), grid, dim3(256), 0, dh::stream(), a);
-    else hipLaunchKernelGGL((attn_prefill_kernel<64, 1>), grid, dim3(256), 0, dh::stream(), a);
+    if (qt == 2) hipLaunchKernelGGL((attn_prefill_kernel<64, 64, 2, false>), grid, dim3(256), 0, dh::stream(), a);
+    else hipLaunchKernelGGL((attn_prefill_kernel<64, 64, 1, false>), grid, dim3(256), 0, dh::stream(), a);
   } else {
-    if (qt == 2) hipLaunchKernelGGL((attn_prefill_kernel<128, 2>), grid, dim3(256), 0, dh::stream(), a);
-    else hipLaunchKernelGGL((attn_prefill_kernel<128, 1>), grid, dim3(256), 0, dh::stream(), a);
+    if (qt == 2) hipLaunchKernelGGL((attn_prefill_kernel<128, 128, 2, false>), grid, dim3(256), 0, dh::stream(), a);
+    else hipLaunchKernelGGL((attn_prefill_kernel<128, 128, 1, false>), grid, dim3(256), 0, dh::stream(), a);
   }
   DH_CHECK_LAUNCH(op);
   return 0;
+}
+
+namespace {
+template <int D, int VD>
+int launch_spec(const char* op, const PrefillArgs& a) {
+  const int qt = dh::ceil_div(a.T, 128) * a.H >= 2 * dh::num_cus() ? 2 : 1;
+  const dim3 grid((unsigned)dh::ceil_div(a.T, 64 * qt), (unsigned)a.H);
+  if (qt == 2) hipLaunchKernelGGL((attn_prefill_kernel<D, VD, 2, true>), grid, dim3(256), 0, dh::stream(), a);
+  else hipLaunchKernelGGL((attn_prefill_kernel<D, VD, 1, true>), grid, dim3(256), 0, dh::stream(), a);
+  DH_CHECK_LAUNCH(op);
+  return 0;
+}
+}  // namespace
+
+extern "C" int dh_attn_spec_prefill(const dh_attn_spec* spec, const float* d_qkv, const void* d_cache_k, const void* d_cache_v,
+                                    void* d_out, int out_dtype, int ld_out, int T, int start_pos) {
+  const char* op = "dh_attn_spec_prefill";
+  DH_REQUIRE_INIT(op);
+  if (int rc = dh::attn_spec_check(op, spec)) return rc;
+  if (T <= 0 || start_pos < 0) return dh::fail(1, "[%s] seqLen must be positive and startPos non-negative", op);
+  if (out_dtype != DH_F32 && out_dtype != DH_BF16) return dh::fail(1, "[%s] output must be f32 or bf16, got dtype %d", op, out_dtype);
+  if (ld_out < spec->H * spec->VD || ld_out % 4) return dh::fail(1, "[%s] ld_out=%d must be a multiple of 4 and hold %d elements", op, ld_out, spec->H * spec->VD);
+  if (!d_qkv || !d_cache_k || !d_cache_v || !d_out) return dh::fail(1, "[%s] null pointer", op);
+  if ((reinterpret_cast<uintptr_t>(d_qkv) | reinterpret_cast<uintptr_t>(d_cache_k) | reinterpret_cast<uintptr_t>(d_cache_v) |
+       reinterpret_cast<uintptr_t>(d_out)) & 15)
+    return dh::fail(1, "[%s] pointers must be 16-byte aligned", op);
+  if (spec->cache_dtype != DH_F16 || spec->D > 128 || spec->VD > 128)
+    return dh::attn_spec_prefill_general(op, spec, d_qkv, d_cache_k, d_cache_v, d_out, out_dtype, ld_out, T, start_pos);
+  PrefillArgs a{};
+  a.Q = d_qkv; a.K = static_cast<const __half*>(d_cache_k); a.V = static_cast<const __half*>(d_cache_v);
+  a.O = out_dtype == DH_F32 ? static_cast<float*>(d_out) : nullptr;
+  a.O16 = out_dtype == DH_BF16 ? static_cast<uint16_t*>(d_out) : nullptr;
+  a.T = T; a.H = spec->H; a.Hkv = spec->Hkv; a.G = spec->H / spec->Hkv; a.kv_len = start_pos + T; a.start_pos = start_pos;
+  a.causal = 1; a.window = spec->window; a.scale = spec->scale; a.softcap = 0.f;
+  a.dk = spec->D; a.dv = spec->VD; a.ld_q = spec->ld_qkv; a.ld_o = ld_out;
+  a.r1 = spec->d_bias_r1; a.r2 = spec->d_bias_r2;
+  a.gate = spec->gate_offset >= 0 ? d_qkv + spec->gate_offset : nullptr;
+  if (spec->D <= 64) return spec->VD <= 64 ? launch_spec<64, 64>(op, a) : launch_spec<64, 128>(op, a);
+  return spec->VD <= 64 ? launch_spec<128, 64>(op, a) : launch_spec<128, 128>(op, a);
 }

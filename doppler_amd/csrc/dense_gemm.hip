@@ -1,0 +1,267 @@
+// Matrix products with dense bf16 weights for several activation rows (prefill).
+//
+//   bf16 activations   v_mfma_f32_32x32x16_bf16, f32 accumulation
+//   f32 activations    v_mfma_f32_32x32x2_f32 on the weights widened (exactly) to f32: a true 32-bit product
+//
+// Weights [N][ldw] and activations [M][lda] are both read along k, 64 elements (bf16) or 32 (f32) at a time; K is
+// a multiple of 64, which the owner of the buffers reaches with zero padding.  A tile of each goes through
+// registers into one of two LDS buffers (loads for the next tile are in flight while the current one is
+// multiplied; one barrier per tile).  LDS rows hold their 16-byte pieces at slot (piece ^ row) & 7, so that both
+// the row-wise stores and the column-wise fragment reads touch every bank once.
+//
+// The epilogue serves two outputs, because the projections that read one normalised row are stored as one
+// stacked matrix: columns below n_first are alpha * acc + bias (+ residual) in f32, columns from n_first on are
+// act(alpha * acc), written in the operand type of the product that reads them.
+#include <algorithm>
+
+#include "dense_device.h"
+
+namespace {
+
+using dh::bf16x8_t;
+using dh::f32x16_t;
+using dh::f32x4_t;
+using dh::u32x4_t;
+
+struct GemmArgs {
+  const void* A;          // [M][lda], bf16 or f32
+  const uint16_t* W;      // [N][ldw] bf16
+  int64_t lda, ldw;
+  int M, N, K;
+  float alpha;
+  const float* bias;      // [n_first] or null
+  const float* residual;  // [M][ldc] or null (may be C)
+  float* C;
+  int64_t ldc;
+  int n_first;
+  void* C2;               // [M][ldc2]
+  int64_t ldc2;
+  int c2_bf16, act;
+  int tiles_m, tiles_n;
+};
+
+// One 32 x 32 accumulator tile: lane l holds column l & 31 and rows 8 (i / 4) + 4 (l >> 5) + i % 4.
+__device__ __forceinline__ void store_tile(const GemmArgs& a, const f32x16_t& acc, int m0, int n0, int lane) {
+  const int n = n0 + (lane & 31);
+  if (n >= a.N) return;
+  const int mb = m0 + 4 * (lane >> 5);
+  if (n < a.n_first) {
+    const float b = a.bias ? a.bias[n] : 0.f;
+#pragma unroll
+    for (int i = 0; i < 16; i++) {
+      const int m = mb + 8 * (i >> 2) + (i & 3);
+      if (m < a.M) {
+        const int64_t at = (int64_t)m * a.ldc + n;
+        float v = fmaf(acc[i], a.alpha, b);
+        if (a.residual) v += a.residual[at];
+        a.C[at] = v;
+      }
+    }
+  } else {
+#pragma unroll
+    for (int i = 0; i < 16; i++) {
+      const int m = mb + 8 * (i >> 2) + (i & 3);
+      if (m < a.M) {
+        const int64_t at = (int64_t)m * a.ldc2 + (n - a.n_first);
+        const float v = dh::activate(acc[i] * a.alpha, a.act);
+        if (a.c2_bf16) static_cast<uint16_t*>(a.C2)[at] = dh::f32_to_bf16_bits(v);
+        else static_cast<float*>(a.C2)[at] = v;
+      }
+    }
+  }
+}
+
+// WM x WN waves; a wave computes TM x TN accumulator tiles of 32 x 32.
+template <int WM, int WN, int TM, int TN>
+__global__ __launch_bounds__(64 * WM * WN) void gemm_bf16_kernel(const GemmArgs a) {
+  constexpr int BM = 32 * WM * TM, BN = 32 * WN * TN, THREADS = 64 * WM * WN;
+  constexpr int PA = BM * 8 / THREADS, PB = BN * 8 / THREADS;      // 16-byte pieces per thread and tile
+  static_assert(BM * 8 % THREADS == 0 && BN * 8 % THREADS == 0, "whole pieces per thread");
+  __shared__ __align__(16) u32x4_t lds[2][(BM + BN) * 8];
+  const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63;
+  const int wm = wave / WN, wn = wave % WN;
+  const int tile = dh::xcd_contiguous(blockIdx.x, a.tiles_m * a.tiles_n);
+  const int m0 = (tile % a.tiles_m) * BM, n0 = (tile / a.tiles_m) * BN;
+
+  // this thread's pieces: rows past the matrix repeat its last row (their products are never stored)
+  const uint16_t* pa[PA];
+  const uint16_t* pb[PB];
+  int sa[PA], sb[PB];
+#pragma unroll
+  for (int r = 0; r < PA; r++) {
+    const int p = tid + THREADS * r, row = p >> 3, c = p & 7;
+    pa[r] = static_cast<const uint16_t*>(a.A) + (int64_t)min(m0 + row, a.M - 1) * a.lda + 8 * c;
+    sa[r] = row * 8 + (c ^ (row & 7));
+  }
+#pragma unroll
+  for (int r = 0; r < PB; r++) {
+    const int p = tid + THREADS * r, row = p >> 3, c = p & 7;
+    pb[r] = a.W + (int64_t)min(n0 + row, a.N - 1) * a.ldw + 8 * c;
+    sb[r] = BM * 8 + row * 8 + (c ^ (row & 7));
+  }
+  u32x4_t ra[PA], rb[PB];
+#define DH_GEMM_LOAD(kt_)                                                                                              \
+  do {                                                                                                                 \
+    _Pragma("unroll") for (int r = 0; r < PA; r++) ra[r] = *reinterpret_cast<const u32x4_t*>(pa[r] + 64 * (kt_));      \
+    _Pragma("unroll") for (int r = 0; r < PB; r++) rb[r] = *reinterpret_cast<const u32x4_t*>(pb[r] + 64 * (kt_));      \
+  } while (0)
+#define DH_GEMM_STORE(b_)                                                                                              \
+  do {                                                                                                                 \
+    _Pragma("unroll") for (int r = 0; r < PA; r++) lds[b_][sa[r]] = ra[r];                                             \
+    _Pragma("unroll") for (int r = 0; r < PB; r++) lds[b_][sb[r]] = rb[r];                                             \
+  } while (0)
+
+  f32x16_t acc[TM][TN];
+#pragma unroll
+  for (int i = 0; i < TM; i++)
+#pragma unroll
+    for (int j = 0; j < TN; j++)
+#pragma unroll
+      for (int e = 0; e < 16; e++) acc[i][j][e] = 0.f;
+
+  const int nk = a.K >> 6;
+  DH_GEMM_LOAD(0);
+  DH_GEMM_STORE(0);
+  __syncthreads();
+  const int frow = lane & 31, fk = lane >> 5;
+  for (int kt = 0; kt < nk; kt++) {
+    const int buf = kt & 1;
+    if (kt + 1 < nk) DH_GEMM_LOAD(kt + 1);
+#pragma unroll
+    for (int ks = 0; ks < 4; ks++) {
+      bf16x8_t fa[TM], fb[TN];
+      const int piece = 2 * ks + fk;
+#pragma unroll
+      for (int i = 0; i < TM; i++) {
+        const int row = 32 * (wm * TM + i) + frow;
+        fa[i] = __builtin_bit_cast(bf16x8_t, lds[buf][row * 8 + (piece ^ (row & 7))]);
+      }
+#pragma unroll
+      for (int j = 0; j < TN; j++) {
+        const int row = 32 * (wn * TN + j) + frow;
+        fb[j] = __builtin_bit_cast(bf16x8_t, lds[buf][BM * 8 + row * 8 + (piece ^ (row & 7))]);
+      }
+#pragma unroll
+      for (int i = 0; i < TM; i++)
+#pragma unroll
+        for (int j = 0; j < TN; j++) acc[i][j] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(fa[i], fb[j], acc[i][j], 0, 0, 0);
+    }
+    if (kt + 1 < nk) DH_GEMM_STORE(buf ^ 1);
+    __syncthreads();
+  }
+#undef DH_GEMM_LOAD
+#undef DH_GEMM_STORE
+#pragma unroll
+  for (int i = 0; i < TM; i++)
+#pragma unroll
+    for (int j = 0; j < TN; j++) store_tile(a, acc[i][j], m0 + 32 * (wm * TM + i), n0 + 32 * (wn * TN + j), lane);
+}
+
+// The 32-bit product: four waves, a 64 x 64 tile, 32 k at a time.  Both tiles sit in LDS as f32 rows of 32 + 4
+// words; a lane reads four consecutive k of its row and feeds four instructions with them (k-slot l >> 5 of
+// instruction e stands for k = 8 s + 4 (l >> 5) + e on both sides).
+__global__ __launch_bounds__(256) void gemm_f32_kernel(const GemmArgs a) {
+  constexpr int BM = 64, BN = 64, BK = 32, ROW = BK + 4;
+  __shared__ __align__(16) float la[BM * ROW];
+  __shared__ __align__(16) float lb[BN * ROW];
+  const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63;
+  const int wm = wave >> 1, wn = wave & 1;
+  const int tile = dh::xcd_contiguous(blockIdx.x, a.tiles_m * a.tiles_n);
+  const int m0 = (tile % a.tiles_m) * BM, n0 = (tile / a.tiles_m) * BN;
+  // A: 64 rows x 8 pieces of 4 floats, two per thread; W: 64 rows x 4 pieces of 8 elements, one per thread
+  const float* pa[2];
+#pragma unroll
+  for (int r = 0; r < 2; r++) {
+    const int p = tid + 256 * r;
+    pa[r] = static_cast<const float*>(a.A) + (int64_t)min(m0 + (p >> 3), a.M - 1) * a.lda + 4 * (p & 7);
+  }
+  const uint16_t* pb = a.W + (int64_t)min(n0 + (tid >> 2), a.N - 1) * a.ldw + 8 * (tid & 3);
+  f32x4_t ra[2];
+  u32x4_t rb;
+  f32x16_t acc;
+#pragma unroll
+  for (int e = 0; e < 16; e++) acc[e] = 0.f;
+  const int nk = a.K / BK;
+#pragma unroll
+  for (int r = 0; r < 2; r++) ra[r] = *reinterpret_cast<const f32x4_t*>(pa[r]);
+  rb = *reinterpret_cast<const u32x4_t*>(pb);
+  for (int kt = 0; kt < nk; kt++) {
+    __syncthreads();
+#pragma unroll
+    for (int r = 0; r < 2; r++) {
+      const int p = tid + 256 * r;
+      *reinterpret_cast<f32x4_t*>(&la[(p >> 3) * ROW + 4 * (p & 7)]) = ra[r];
+    }
+    float* wb = &lb[(tid >> 2) * ROW + 8 * (tid & 3)];
+#pragma unroll
+    for (int e = 0; e < 4; e++) {
+      wb[2 * e] = dh::bf16_low(rb[e]);
+      wb[2 * e + 1] = dh::bf16_high(rb[e]);
+    }
+    __syncthreads();
+    if (kt + 1 < nk) {
+#pragma unroll
+      for (int r = 0; r < 2; r++) ra[r] = *reinterpret_cast<const f32x4_t*>(pa[r] + BK * (kt + 1));
+      rb = *reinterpret_cast<const u32x4_t*>(pb + BK * (kt + 1));
+    }
+#pragma unroll
+    for (int s = 0; s < BK / 8; s++) {
+      const int k = 8 * s + 4 * (lane >> 5);
+      const f32x4_t fa = *reinterpret_cast<const f32x4_t*>(&la[(32 * wm + (lane & 31)) * ROW + k]);
+      const f32x4_t fb = *reinterpret_cast<const f32x4_t*>(&lb[(32 * wn + (lane & 31)) * ROW + k]);
+#pragma unroll
+      for (int e = 0; e < 4; e++) acc = __builtin_amdgcn_mfma_f32_32x32x2f32(fa[e], fb[e], acc, 0, 0, 0);
+    }
+  }
+  store_tile(a, acc, m0 + 32 * wm, n0 + 32 * wn, lane);
+}
+
+template <int WM, int WN, int TM, int TN>
+int launch_bf16(const char* op, GemmArgs a) {
+  a.tiles_m = (int)dh::ceil_div(a.M, 32 * WM * TM);
+  a.tiles_n = (int)dh::ceil_div(a.N, 32 * WN * TN);
+  hipLaunchKernelGGL((gemm_bf16_kernel<WM, WN, TM, TN>), dim3(a.tiles_m * a.tiles_n), dim3(64 * WM * WN), 0, dh::stream(), a);
+  DH_CHECK_LAUNCH(op);
+  return 0;
+}
+
+}  // namespace
+
+extern "C" int dh_dense_matmul(const void* d_A, int a_dtype, int lda, const void* d_W, int ldw, int M, int N, int K,
+                               float alpha, const float* d_bias, const float* d_residual, float* d_C, int ldc, int n_first,
+                               void* d_C2, int c2_dtype, int ldc2, int activation) {
+  const char* op = "dh_dense_matmul";
+  DH_REQUIRE_INIT(op);
+  if (M <= 0 || N <= 0 || K <= 0) return dh::fail(1, "[%s] Dimensions must be positive: M=%d, N=%d, K=%d", op, M, N, K);
+  if (K % 64) return dh::fail(1, "[%s] K=%d must be a multiple of 64 (zero-padded)", op, K);
+  if (lda < K || ldw < K || lda % 8 || ldw % 8)
+    return dh::fail(1, "[%s] row strides must be multiples of 8 and hold K=%d elements (lda=%d, ldw=%d)", op, K, lda, ldw);
+  if (a_dtype != DH_BF16 && a_dtype != DH_F32) return dh::fail(1, "[%s] activations must be bf16 or f32, got dtype %d", op, a_dtype);
+  if (n_first < 0 || n_first > N) return dh::fail(1, "[%s] n_first=%d is outside 0..%d", op, n_first, N);
+  if (!d_A || !d_W || (n_first > 0 && !d_C) || (n_first < N && !d_C2)) return dh::fail(1, "[%s] null pointer", op);
+  if (n_first > 0 && ldc < n_first) return dh::fail(1, "[%s] ldc=%d is shorter than %d columns", op, ldc, n_first);
+  if (n_first < N && (ldc2 < N - n_first || (c2_dtype != DH_BF16 && c2_dtype != DH_F32)))
+    return dh::fail(1, "[%s] the second output needs %d columns of bf16 or f32 (ldc2=%d, dtype %d)", op, N - n_first, ldc2, c2_dtype);
+  if ((reinterpret_cast<uintptr_t>(d_A) | reinterpret_cast<uintptr_t>(d_W)) & 15)
+    return dh::fail(1, "[%s] activation and weight pointers must be 16-byte aligned", op);
+  GemmArgs a{};
+  a.A = d_A; a.W = static_cast<const uint16_t*>(d_W); a.lda = lda; a.ldw = ldw;
+  a.M = M; a.N = N; a.K = K; a.alpha = alpha; a.bias = d_bias; a.residual = d_residual;
+  a.C = d_C; a.ldc = ldc; a.n_first = n_first;
+  a.C2 = d_C2; a.ldc2 = ldc2; a.c2_bf16 = c2_dtype == DH_BF16; a.act = activation;
+  if (a_dtype == DH_F32) {
+    a.tiles_m = (int)dh::ceil_div(M, 64);
+    a.tiles_n = (int)dh::ceil_div(N, 64);
+    hipLaunchKernelGGL(gemm_f32_kernel, dim3(a.tiles_m * a.tiles_n), dim3(256), 0, dh::stream(), a);
+    DH_CHECK_LAUNCH(op);
+    return 0;
+  }
+  // the largest tile that still gives every compute unit work
+  const int cus = dh::num_cus();
+  auto tiles = [&](int bm, int bn) { return dh::ceil_div(M, bm) * dh::ceil_div(N, bn); };
+  static const int env_tile = dh::tuning_int("DH_DENSE_TILE", 0);
+  const int pick = env_tile ? env_tile : tiles(256, 256) >= cus ? 256 : tiles(128, 128) >= cus ? 128 : 64;
+  if (pick == 256) return launch_bf16<2, 4, 4, 2>(op, a);
+  if (pick == 128) return launch_bf16<2, 2, 2, 2>(op, a);
+  return launch_bf16<2, 2, 1, 1>(op, a);
+}

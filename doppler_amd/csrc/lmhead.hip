@@ -10,45 +10,16 @@
 #include <algorithm>
 #include <cfloat>
 
+#include "argmax_device.h"
 #include "dh_common.h"
 
 namespace {
 
-constexpr int kMaxParts = 2048;
-
-struct Cand {
-  float v;
-  uint32_t i;
-};
-
-__device__ __forceinline__ bool beats(float cv, uint32_t ci, float bv, uint32_t bi) {
-  if (cv > bv) return true;
-  if (cv < bv) return false;
-  return ci < bi;
-}
-
-__device__ __forceinline__ Cand wave_best(Cand c) {
-#pragma unroll
-  for (int off = 32; off > 0; off >>= 1) {
-    const float ov = __shfl_xor(c.v, off, 64);
-    const uint32_t oi = __shfl_xor(c.i, off, 64);
-    if (beats(ov, oi, c.v, c.i)) { c.v = ov; c.i = oi; }
-  }
-  return c;
-}
-
-// Workgroup-wide best of 256 threads; valid in thread 0.
-__device__ __forceinline__ Cand block_best_256(Cand c, float* sv, uint32_t* si) {
-  c = wave_best(c);
-  const int wave = threadIdx.x >> 6;
-  if ((threadIdx.x & 63) == 0) { sv[wave] = c.v; si[wave] = c.i; }
-  __syncthreads();
-  if (threadIdx.x == 0) {
-    for (int w = 1; w < 4; w++)
-      if (beats(sv[w], si[w], c.v, c.i)) { c.v = sv[w]; c.i = si[w]; }
-  }
-  return c;
-}
+using dh::Cand;
+using dh::beats;
+using dh::block_best_256;
+using dh::stream_load_16;
+using dh::kMaxParts;
 
 __device__ __forceinline__ float softcap_f(float x, float cap) {
   return cap > 0.f ? cap * tanhf(x / cap) : x;
@@ -71,17 +42,6 @@ struct F16GemvArgs {
   float norm_eps;
   int norm_weight_offset;
 };
-
-// 16 bytes of a weight row, marked non-temporal.  Every row is read once per call, by one wave, as whole
-// cache lines (a wave's load covers 1 KB of consecutive bytes): with the streaming hint the [151936 x 4096]
-// f16 head is read at 6.6 TB/s against 5.9 TB/s with ordinary loads.  (The same hint on loads whose cache
-// lines are shared between waves, the Q4_K units' 144-byte row pieces and the decode attention's K/V rows,
-// made those kernels slower.)
-__device__ __forceinline__ uint4 stream_load_16(const uint4* p) {
-  typedef uint32_t u32x4 __attribute__((ext_vector_type(4)));
-  const u32x4 t = __builtin_nontemporal_load(reinterpret_cast<const u32x4*>(p));
-  return make_uint4(t[0], t[1], t[2], t[3]);
-}
 
 // M = 1, K <= 4096: every lane meets the same 64 activations in every row (its eight 16-byte
 // chunks sit at fixed k), so they live in registers for the whole kernel; LDS only hands the row to
@@ -325,6 +285,15 @@ int check_f16w_shape(const char* op, int M, int N, int K) {
 }
 
 }  // namespace
+
+namespace dh {
+int launch_argmax_final(const char* op, const float* part_val, const uint32_t* part_idx, int parts, uint32_t* token_out,
+                        int out_index) {
+  hipLaunchKernelGGL(argmax_final_kernel, dim3(1), dim3(256), 0, stream(), part_val, part_idx, parts, token_out, out_index);
+  DH_CHECK_LAUNCH(op);
+  return 0;
+}
+}  // namespace dh
 
 extern "C" {
 

@@ -35,9 +35,12 @@ extern "C" {
 
 #define DH_F32 0
 #define DH_F16 1
+#define DH_BF16 2
 
 #define DH_ACT_SILU 0
 #define DH_ACT_GELU 1
+#define DH_ACT_RELU2 2   /* max(z, 0)^2: plain activations of the dense products only */
+#define DH_ACT_NONE (-1)
 
 #define DH_KV_CONTIGUOUS 0
 #define DH_KV_RING 1
@@ -351,6 +354,80 @@ int dh_attn_decode_qkv_kvlen_partials(const float* d_qkv, const float* d_q_weigh
                                       int max_kv_len, int rotary_dim, int interleaved, float eps,
                                       int weight_offset, int use_norm, float scale, float softcap,
                                       int sliding_window, int kv_start, int kv_layout, void* d_workspace);
+
+/* ---- dense bf16 weights (models whose linear layers are not quantised) ----
+ * No counterpart in the reference's Q4_K path.  Weights are bf16 rows [N][ldw], applied as W x; K is a multiple
+ * of 64 and the rows of W and of the activations are zero-padded to it.  Two compute types: bf16 activations
+ * (matrix cores, f32 accumulation) or f32 activations (a true 32-bit product, the weights widened exactly).
+ *
+ * Projections that read the same row are stored stacked and run as one product with two outputs: column
+ * n < n_first is  C[m][n] = alpha * acc + bias[n] + residual[m][n]  (f32; bias and residual may be NULL, residual has
+ * C's stride and may be C itself), column n >= n_first is  C2[m][n - n_first] = act(alpha * acc)  in c2_dtype
+ * (DH_BF16 or DH_F32).  n_first = N: no second output. */
+int dh_dense_matmul(const void* d_A, int a_dtype, int lda, const void* d_W, int ldw, int M, int N, int K, float alpha,
+                    const float* d_bias, const float* d_residual, float* d_C, int ldc, int n_first, void* d_C2,
+                    int c2_dtype, int ldc2, int activation);
+
+/* The same product for ONE f32 activation row (decode; HBM-bound), d_C2 in f32, with an optional RMSNorm of the
+ * row in its prologue: x * rsqrt(mean of the first `hidden` elements squared + eps) * w.  d_x and d_norm_weight
+ * hold K elements (zero from `hidden` on); K <= 32768. */
+int dh_dense_gemv(const float* d_x, const float* d_norm_weight, int hidden, float eps, const void* d_W, int ldw, int N,
+                  int K, float alpha, const float* d_bias, const float* d_residual, float* d_C, int n_first, float* d_C2,
+                  int activation);
+/* dh_lmhead_argmax_f16_rmsnorm for an untied bf16 head: logits = alpha * W norm(x), token = their argmax (ties to
+ * the lowest index).  d_workspace: dh_lmhead_argmax_workspace_bytes(vocab). */
+int dh_dense_lmhead_argmax(const float* d_x, const float* d_norm_weight, int hidden, float eps, const void* d_W, int ldw,
+                           int vocab, int K, float alpha, void* d_workspace, uint32_t* d_token_out, int output_index,
+                           float* d_logits_out);
+
+/* out[t] = embed[id_t] + bigram[row_t] + pos[p_t], bf16 tables of `hidden` columns, f32 sum; p_t = start_pos + t, or
+ * with d_kv_len (key count on the device, T = 1) *d_kv_len - 1.  row_t = (id_{t-1} * mul_prev + id_t * mul_cur) mod
+ * buckets, or `buckets` (the table's last row) at position 0; the token before the first is *d_prev.  d_bigram and
+ * d_pos may be NULL (no such term).  Output rows are ld_out floats apart.  Ids outside the vocabulary and positions
+ * outside the table contribute zero rows. */
+int dh_embed_sum(const uint32_t* d_ids, int index_offset, const uint32_t* d_prev, const void* d_embed, int vocab,
+                 const void* d_bigram, int64_t buckets, int64_t mul_prev, int64_t mul_cur, const void* d_pos,
+                 int max_positions, float* d_out, int ld_out, int T, int hidden, int start_pos, const uint32_t* d_kv_len);
+
+/* RMSNorm of n rows into the operand type of the product that reads them: out[r] = norm(x[rows ? rows[r] : r]),
+ * columns hidden .. ld_out - 1 zero.  out_dtype DH_BF16 or DH_F32. */
+int dh_rmsnorm_rows(const float* d_x, int ld_x, const uint32_t* d_rows, const float* d_weight, void* d_out, int out_dtype,
+                    int ld_out, int n, int hidden, float eps);
+
+/* ---- attention with a distance bias, an output gate and separate key and value sizes ----
+ * One layer's attention of a decoder without rotary positions:
+ *   score_ij = scale * q_i . k_j - bias_r1[h] * ln(1 + bias_r2[h] * (i - j)),  softmax over 0 <= i - j < window,
+ *   out_i    = sigmoid(gate_i[h]) * sum_j softmax_ij * value_j
+ * window 0: all earlier keys.  bias_r1/r2 NULL: no bias; gate offset < 0: no gate; value_norm: each head's value is
+ * divided by its root mean square over value_dim (value_eps inside the root) before it is cached.
+ * Head sizes D (keys) and VD (values) are the padded ones, multiples of 8 up to 512, whose padding holds zeros; value_dim is the number
+ * of real value elements.  Caches are [row][Hkv][D] and [row][Hkv][VD], f16 or f32 (cache_dtype), one row per position.
+ * A step's projections are rows of ld_qkv floats with q heads at 0, k heads at k_offset, v heads at v_offset and the H gate
+ * numbers at gate_offset. */
+typedef struct dh_attn_spec {
+  int H, Hkv, D, VD, value_dim;
+  int window;
+  int cache_dtype;
+  int value_norm;
+  int k_offset, v_offset, gate_offset, ld_qkv;
+  float scale, value_eps;
+  const float* d_bias_r1;   /* [H] */
+  const float* d_bias_r2;   /* [H] */
+} dh_attn_spec;
+/* Keys and (normed) values of T projection rows into the caches at rows start_pos .. start_pos + T - 1. */
+int dh_attn_spec_kv_write(const dh_attn_spec* spec, const float* d_qkv, void* d_cache_k, void* d_cache_v, int T,
+                          int start_pos);
+/* T queries at positions start_pos .. against the cache rows up to their own (already written).  Output rows of H * VD
+ * elements, ld_out apart, f32 or bf16.  f16 caches with D, VD <= 128 run on the matrix cores. */
+int dh_attn_spec_prefill(const dh_attn_spec* spec, const float* d_qkv, const void* d_cache_k, const void* d_cache_v,
+                         void* d_out, int out_dtype, int ld_out, int T, int start_pos);
+/* One step from its raw projection row: key and value are appended at row `pos`, the token attends to its window;
+ * d_out is [H * VD] f32.  d_kv_len (may be NULL): the key count pos + 1 is read from device memory instead, at most
+ * max_kv_len (a captured step then replays at every position).  d_workspace: dh_attn_spec_workspace_bytes(H, VD,
+ * max_kv_len or pos + 1). */
+size_t dh_attn_spec_workspace_bytes(int H, int VD, int max_kv_len);
+int dh_attn_spec_decode(const dh_attn_spec* spec, const float* d_qkv, void* d_cache_k, void* d_cache_v, float* d_out,
+                        int pos, const uint32_t* d_kv_len, int max_kv_len, void* d_workspace);
 
 /* ---- normalisation / rotary / KV ---- */
 
