@@ -12,6 +12,7 @@ through the C ABI, one 4-byte token readback per step.  Prints ONE JSON line wit
   cpu_baseline  the CPU oracle's decode step timed on this host's cores on a bounded sample.
 
     python bench.py [--gpus 1] [--steps K] [--warmup W]
+    python bench.py --design zepavik [--sizes 1024,2048,4096]     # that design beside the Q4_K decoder at equal size
 """
 import argparse
 import ctypes
@@ -172,6 +173,9 @@ def main():
     ap.add_argument("--copy-calibration", action="store_true",
                     help="also run three f32->f16 casts of 16 Mi elements (64 MiB read, 32 MiB written): a "
                          "streaming kernel of known traffic to scale rocprofv3 FETCH_SIZE / WRITE_SIZE with")
+    ap.add_argument("--design", choices=("zepavik",), default=None,
+                    help="measure this design's prefill, decode and kernels beside the Q4_K decoder instead")
+    ap.add_argument("--sizes", default="1024,2048,4096", help="with --design: widths to measure")
     args = ap.parse_args()
     if args.gpus != 1:
         print("bench.py: this build runs on ONE GPU (single-stream decode has nothing to shard in this tier); "
@@ -185,6 +189,19 @@ def main():
     if not torch.cuda.is_available():
         print("bench.py: no GPU visible; the HIP path has no CPU fallback", file=sys.stderr)
         sys.exit(1)
+
+    if args.design:
+        from doppler_amd import design_bench
+        sizes = args.sizes.split(",")
+        res = design_bench.run(sizes, args.steps, args.warmup)
+        last = res[sizes[-1]]
+        print(json.dumps({"metric": "decode tokens/sec, %s at width %s, 1 GPU" % (args.design, sizes[-1]),
+                          "value": last[args.design]["decode_tokens_per_s"], "unit": "tokens/s", "n_gpus": 1, "steps": args.steps,
+                          "warmup": args.warmup, "ms_per_step": round(1e3 / last[args.design]["decode_tokens_per_s"], 4),
+                          "higher_is_better": True, "scaling": "weak", "vs_baseline": None,
+                          "dtype": "bf16 weights and matrix-core operands, f32 residual, norms, scores and decode activations, f16 KV cache",
+                          "data": "synthetic", "config": res}), flush=True)
+        return
 
     c = dict(synth.CFG4)
     prefill, _ = c.pop("prefill"), c.pop("steps")

@@ -80,7 +80,7 @@ struct PrefillArgs {
 // QT = 16-query groups per wave: every K and V fragment read from LDS feeds QT matrix-core
 // instructions, and a workgroup tile (64 QT queries) stages each key tile once.
 template <int D, int VD, int QT, bool SPEC>
-__global__ __launch_bounds__(256) void attn_prefill_kernel(const PrefillArgs a) {
+__global__ __launch_bounds__(256, SPEC ? 2 : 1) void attn_prefill_kernel(const PrefillArgs a) {
   constexpr int BQ = 64 * QT;
   constexpr int STEPS = D / 32;            // MFMAs per 16 x 16 score tile
   constexpr int DT = VD / 16;              // output row tiles (of O^T)
@@ -367,7 +367,8 @@ extern "C" int dh_attn_prefill(const float* d_Q, const void* d_K, const void* d_
 namespace {
 template <int D, int VD>
 int launch_spec(const char* op, const PrefillArgs& a) {
-  const int qt = dh::ceil_div(a.T, 128) * a.H >= 2 * dh::num_cus() ? 2 : 1;
+  static const int env_qt = dh::tuning_int("DH_ATTN_SPEC_QT", 0);
+  const int qt = env_qt ? env_qt : dh::ceil_div(a.T, 128) * a.H >= 2 * dh::num_cus() ? 2 : 1;
   const dim3 grid((unsigned)dh::ceil_div(a.T, 64 * qt), (unsigned)a.H);
   if (qt == 2) hipLaunchKernelGGL((attn_prefill_kernel<D, VD, 2, true>), grid, dim3(256), 0, dh::stream(), a);
   else hipLaunchKernelGGL((attn_prefill_kernel<D, VD, 1, true>), grid, dim3(256), 0, dh::stream(), a);

@@ -12,6 +12,9 @@
 // The epilogue serves two outputs, because the projections that read one normalised row are stored as one
 // stacked matrix: columns below n_first are alpha * acc + bias (+ residual) in f32, columns from n_first on are
 // act(alpha * acc), written in the operand type of the product that reads them.
+//
+// A grid of too few tiles for the device cuts k into slices instead (grid.y): every slice leaves its raw sums in the
+// library's split-K workspace and a second launch adds them in slice order and runs the epilogue.
 #include <algorithm>
 
 #include "dense_device.h"
@@ -38,36 +41,43 @@ struct GemmArgs {
   int64_t ldc2;
   int c2_bf16, act;
   int tiles_m, tiles_n;
+  float* parts;           // [slices][M][N] raw sums instead of the outputs, or null
+  int k_slice;            // k extent of a slice (a multiple of 64); K when there is one
 };
+
+// The two outputs of one element.
+__device__ __forceinline__ void put(const GemmArgs& a, int m, int n, float acc) {
+  if (n < a.n_first) {
+    const int64_t at = (int64_t)m * a.ldc + n;
+    float v = fmaf(acc, a.alpha, a.bias ? a.bias[n] : 0.f);
+    if (a.residual) v += a.residual[at];
+    a.C[at] = v;
+  } else {
+    const int64_t at = (int64_t)m * a.ldc2 + (n - a.n_first);
+    const float v = dh::activate(acc * a.alpha, a.act);
+    if (a.c2_bf16) static_cast<uint16_t*>(a.C2)[at] = dh::f32_to_bf16_bits(v);
+    else static_cast<float*>(a.C2)[at] = v;
+  }
+}
 
 // One 32 x 32 accumulator tile: lane l holds column l & 31 and rows 8 (i / 4) + 4 (l >> 5) + i % 4.
 __device__ __forceinline__ void store_tile(const GemmArgs& a, const f32x16_t& acc, int m0, int n0, int lane) {
   const int n = n0 + (lane & 31);
   if (n >= a.N) return;
   const int mb = m0 + 4 * (lane >> 5);
-  if (n < a.n_first) {
-    const float b = a.bias ? a.bias[n] : 0.f;
+  if (a.parts) {
+    float* p = a.parts + (int64_t)blockIdx.y * a.M * a.N;
 #pragma unroll
     for (int i = 0; i < 16; i++) {
       const int m = mb + 8 * (i >> 2) + (i & 3);
-      if (m < a.M) {
-        const int64_t at = (int64_t)m * a.ldc + n;
-        float v = fmaf(acc[i], a.alpha, b);
-        if (a.residual) v += a.residual[at];
-        a.C[at] = v;
-      }
+      if (m < a.M) p[(int64_t)m * a.N + n] = acc[i];
     }
-  } else {
+    return;
+  }
 #pragma unroll
-    for (int i = 0; i < 16; i++) {
-      const int m = mb + 8 * (i >> 2) + (i & 3);
-      if (m < a.M) {
-        const int64_t at = (int64_t)m * a.ldc2 + (n - a.n_first);
-        const float v = dh::activate(acc[i] * a.alpha, a.act);
-        if (a.c2_bf16) static_cast<uint16_t*>(a.C2)[at] = dh::f32_to_bf16_bits(v);
-        else static_cast<float*>(a.C2)[at] = v;
-      }
-    }
+  for (int i = 0; i < 16; i++) {
+    const int m = mb + 8 * (i >> 2) + (i & 3);
+    if (m < a.M) put(a, m, n, acc[i]);
   }
 }
 
@@ -119,7 +129,12 @@ __global__ __launch_bounds__(64 * WM * WN) void gemm_bf16_kernel(const GemmArgs 
 #pragma unroll
       for (int e = 0; e < 16; e++) acc[i][j][e] = 0.f;
 
-  const int nk = a.K >> 6;
+  const int k0 = blockIdx.y * a.k_slice;
+  const int nk = min(a.k_slice, a.K - k0) >> 6;
+#pragma unroll
+  for (int r = 0; r < PA; r++) pa[r] += k0;
+#pragma unroll
+  for (int r = 0; r < PB; r++) pb[r] += k0;
   DH_GEMM_LOAD(0);
   DH_GEMM_STORE(0);
   __syncthreads();
@@ -216,12 +231,34 @@ __global__ __launch_bounds__(256) void gemm_f32_kernel(const GemmArgs a) {
   store_tile(a, acc, m0 + 32 * wm, n0 + 32 * wn, lane);
 }
 
+__global__ __launch_bounds__(256) void gemm_reduce_kernel(const GemmArgs a, int slices) {
+  const int64_t total = (int64_t)a.M * a.N;
+  for (int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x; i < total; i += (int64_t)gridDim.x * 256) {
+    float s = 0.f;
+#pragma unroll 4
+    for (int k = 0; k < slices; k++) s += a.parts[k * total + i];
+    put(a, (int)(i / a.N), (int)(i % a.N), s);
+  }
+}
+
 template <int WM, int WN, int TM, int TN>
-int launch_bf16(const char* op, GemmArgs a) {
+int launch_bf16(const char* op, GemmArgs a, int slices) {
   a.tiles_m = (int)dh::ceil_div(a.M, 32 * WM * TM);
   a.tiles_n = (int)dh::ceil_div(a.N, 32 * WN * TN);
-  hipLaunchKernelGGL((gemm_bf16_kernel<WM, WN, TM, TN>), dim3(a.tiles_m * a.tiles_n), dim3(64 * WM * WN), 0, dh::stream(), a);
+  a.k_slice = a.K;
+  if (slices > 1) {
+    a.k_slice = (int)dh::ceil_div(a.K / 64, slices) * 64;
+    slices = (int)dh::ceil_div(a.K, a.k_slice);
+    size_t bytes = 0;
+    a.parts = dh::splitk_workspace(&bytes);
+  }
+  hipLaunchKernelGGL((gemm_bf16_kernel<WM, WN, TM, TN>), dim3(a.tiles_m * a.tiles_n, slices), dim3(64 * WM * WN), 0, dh::stream(), a);
   DH_CHECK_LAUNCH(op);
+  if (a.parts) {
+    const unsigned grid = (unsigned)std::min<int64_t>(dh::ceil_div((int64_t)a.M * a.N, 256), 4096);
+    hipLaunchKernelGGL(gemm_reduce_kernel, dim3(grid), dim3(256), 0, dh::stream(), a, slices);
+    DH_CHECK_LAUNCH(op);
+  }
   return 0;
 }
 
@@ -256,12 +293,21 @@ extern "C" int dh_dense_matmul(const void* d_A, int a_dtype, int lda, const void
     DH_CHECK_LAUNCH(op);
     return 0;
   }
-  // the largest tile that still gives every compute unit work
+  // 128 x 128 tiles (two workgroups per compute unit) where they fill the device, 64 x 64 otherwise.  (256 x 256 and
+  // 256 x 128 tiles measured the same or slower at every shape tried: one workgroup per compute unit hides less.)
   const int cus = dh::num_cus();
   auto tiles = [&](int bm, int bn) { return dh::ceil_div(M, bm) * dh::ceil_div(N, bn); };
   static const int env_tile = dh::tuning_int("DH_DENSE_TILE", 0);
-  const int pick = env_tile ? env_tile : tiles(256, 256) >= cus ? 256 : tiles(128, 128) >= cus ? 128 : 64;
-  if (pick == 256) return launch_bf16<2, 4, 4, 2>(op, a);
-  if (pick == 128) return launch_bf16<2, 2, 2, 2>(op, a);
-  return launch_bf16<2, 2, 1, 1>(op, a);
+  static const int env_slices = dh::tuning_int("DH_DENSE_SLICES", 0);
+  // slices of at least 1024 k, as many as fill the device, within the workspace
+  size_t ws_bytes = 0;
+  (void)dh::splitk_workspace(&ws_bytes);
+  const int64_t most = std::max<int64_t>(1, std::min<int64_t>(K / 1024, (int64_t)(ws_bytes / ((size_t)M * N * sizeof(float)))));
+  auto slices_for = [&](int64_t t, int per_cu) { return std::min(most, std::max<int64_t>(1, (int64_t)per_cu * cus / t)); };
+  const bool big_enough = tiles(128, 128) >= cus || (M > 64 && tiles(128, 128) * most >= cus);
+  const int pick = env_tile ? env_tile : big_enough ? 128 : 64;
+  const int64_t t = tiles(pick, pick);
+  const int slices = env_slices ? (int)std::min<int64_t>(env_slices, most) : t >= cus ? 1 : (int)slices_for(t, pick == 128 ? 2 : 4);
+  if (pick == 128) return launch_bf16<2, 2, 2, 2>(op, a, slices);
+  return launch_bf16<2, 2, 1, 1>(op, a, slices);
 }

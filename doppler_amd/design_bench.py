@@ -1,0 +1,203 @@
+"""Throughput of a design beside the closest decoder the package serves, at sizes that resemble a real model's layers.
+
+Zepavik (dense bf16, parallel layers, windowed attention) against the Q4_K decoder with the same width, heads, feed-forward
+width and layer count: prefill and decode tokens/s, and per kernel the share of its roofline (8 TB/s of HBM, 2.5
+PFLOP/s on the matrix cores).  Random weights; kernels cycle through more weights than the caches hold.
+"""
+import ctypes
+import sys
+import time
+
+import numpy as np
+
+HBM_GBPS, MFMA_TFLOPS = 8000.0, 2500.0
+SIZES = {
+    "1024": dict(hidden=1024, heads=16, kv_heads=8, head_dim=64, ff=3072, layers=24),
+    "2048": dict(hidden=2048, heads=16, kv_heads=8, head_dim=128, ff=6144, layers=12),
+    "4096": dict(hidden=4096, heads=32, kv_heads=8, head_dim=128, ff=12288, layers=6),
+}
+VOCAB, WINDOW, PROMPT = 32000, 1024, 2048
+
+
+def log(*a):
+    print(*a, file=sys.stderr, flush=True)
+
+
+def zepavik_config(s, max_seq):
+    mixer = dict(heads=s["heads"], kv_heads=s["kv_heads"], dim=s["head_dim"], vdim=s["head_dim"], window=WINDOW,
+                 scale=s["head_dim"] ** -0.5, log_bias=True, value_norm=True, gate=True)
+    return dict(hidden=s["hidden"], vocab=VOCAB, eps=1e-5, logit_scale=1.0, max_positions=max_seq,
+                bigram=dict(buckets=4096, mul_prev=31, mul_cur=7),
+                layers=[dict(mixer=dict(mixer), mlp=dict(ff=s["ff"], activation="relu2")) for _ in range(s["layers"])])
+
+
+def q4k_config(s, max_seq):
+    return dict(layers=s["layers"], hidden=s["hidden"], inter=s["ff"], heads=s["heads"], kv_heads=s["kv_heads"],
+                head_dim=s["head_dim"], vocab=VOCAB, eps=1e-6, qk_norm=1, theta=1e6, max_seq=max_seq)
+
+
+class _Timer:
+    def __init__(self, L):
+        from . import capi
+        self.L, self.ck = L, capi.check
+        self.ev = [ctypes.c_void_p() for _ in range(2)]
+        for e in self.ev:
+            self.ck(L.dh_event_create(ctypes.byref(e)))
+
+    def us(self, calls, reps=3):
+        """Fastest sweep over the calls, per call."""
+        for c in calls:
+            c()
+        self.ck(self.L.dh_sync())
+        best = float("inf")
+        for _ in range(reps):
+            self.ck(self.L.dh_event_record(self.ev[0]))
+            for c in calls:
+                c()
+            self.ck(self.L.dh_event_record(self.ev[1]))
+            ms = ctypes.c_float()
+            self.ck(self.L.dh_event_elapsed_ms(self.ev[0], self.ev[1], ctypes.byref(ms)))
+            best = min(best, ms.value / len(calls))
+        return best * 1e3
+
+    def close(self):
+        for e in self.ev:
+            self.ck(self.L.dh_event_destroy(e))
+
+
+def _throughput(dec, prompt, steps, warmup):
+    """(prefill tokens/s, decode tokens/s) of a decoder through its own prefill and generation loop."""
+    dec.prefill(prompt, chunk=PROMPT)
+    dec.L.dh_sync()
+    t0 = time.perf_counter()
+    tok = dec.prefill(prompt, chunk=PROMPT)
+    dec.L.dh_sync()
+    prefill = len(prompt) / (time.perf_counter() - t0)
+    out = dec.decode_greedy(tok, len(prompt), max(warmup, 1))
+    dec.L.dh_sync()
+    t0 = time.perf_counter()
+    dec.decode_greedy(out[-1], len(prompt) + len(out), steps)
+    dec.L.dh_sync()
+    decode = steps / (time.perf_counter() - t0)
+    dec.release_readback()
+    return prefill, decode
+
+
+def _entry(name, us, nbytes=None, flops=None):
+    e = dict(kernel=name, us=round(us, 2))
+    if nbytes is not None:
+        e.update(gb_per_s=round(nbytes / us / 1e3, 1), hbm_frac=round(nbytes / us / 1e3 / HBM_GBPS, 4))
+    else:
+        e.update(tflop_per_s=round(flops / us / 1e6, 1), mfma_frac=round(flops / us / 1e6 / MFMA_TFLOPS, 4))
+    return e
+
+
+def _attn_flops(T, heads, dim, window):
+    pairs = sum(min(t + 1, window) if window else t + 1 for t in range(T))
+    return 4.0 * pairs * heads * dim
+
+
+def zepavik_kernels(dec, s, T):
+    from . import capi
+    L, ck, c = dec.L, capi.check, dec.cfg
+    t, pos = _Timer(L), PROMPT + 8
+    Hd, g = c["hidden"], dec.layers[0]["geo"]
+    mixed = dec.mixed[dec._mixed_key(g)].data_ptr()
+    act = mixed + 4 * g["attn_cols"]
+    b = dec._pf
+    pm, x, qkv = b["mixed"][dec._mixed_key(g)].data_ptr(), b["x"].data_ptr(), b["qkv"].data_ptr()
+    elem = b["normed"].element_size()
+    out = []
+    sweep = lambda f: t.us([(lambda d=d: f(d)) for d in dec.layers])
+    us = sweep(lambda d: ck(L.dh_dense_gemv(dec.x.data_ptr(), d["norm"].data_ptr(), Hd, c["eps"], d["w_in"].data_ptr(), g["kx"], g["n"],
+                                            g["kx"], 1.0, d["bias"].data_ptr(), None, dec.qkv.data_ptr(), g["n_first"], act, d["act"])))
+    out.append(_entry("decode: norm + q/k/v/gate/up", us, nbytes=2.0 * g["n"] * Hd))
+    us = sweep(lambda d: ck(L.dh_dense_gemv(mixed, None, 0, 0.0, d["w_out"].data_ptr(), g["k2"], Hd, g["k2"], 1.0, None,
+                                            dec.x.data_ptr(), dec.x.data_ptr(), Hd, None, capi.ACT_NONE)))
+    out.append(_entry("decode: o/down + residual", us, nbytes=2.0 * Hd * (g["attn_cols"] + g["ff"])))
+    us = sweep(lambda d: ck(L.dh_attn_spec_decode(ctypes.byref(d["spec"]), dec.qkv.data_ptr(), d["cache_k"].data_ptr(),
+                                                  d["cache_v"].data_ptr(), mixed, pos, None, 0, dec.attn_ws.data_ptr())))
+    out.append(_entry("decode: attention, %d keys" % WINDOW, us, nbytes=2.0 * WINDOW * s["kv_heads"] * (g["D"] + g["VD"])))
+    us = sweep(lambda d: ck(L.dh_dense_lmhead_argmax(dec.x.data_ptr(), dec.final_norm.data_ptr(), Hd, c["eps"], dec.head.data_ptr(),
+                                                     dec.kx, c["vocab"], dec.kx, 1.0, dec.lm_ws.data_ptr(), dec.token.data_ptr(), 0, None)))
+    out.append(_entry("decode: norm + head + argmax (weights in cache where they fit)", us, nbytes=2.0 * c["vocab"] * Hd))
+    us = sweep(lambda d: dec._enqueue_in(d, x, b["normed"].data_ptr(), dec.operand, qkv, pm + elem * g["attn_cols"], T, g["k2"]))
+    out.append(_entry("prefill: norm, q/k/v/gate/up", us, flops=2.0 * T * g["n"] * Hd))
+    us = sweep(lambda d: dec._enqueue_out(d, pm, dec.operand, x, T))
+    out.append(_entry("prefill: o/down + residual", us, flops=2.0 * T * Hd * (g["attn_cols"] + g["ff"])))
+    us = sweep(lambda d: ck(L.dh_attn_spec_prefill(ctypes.byref(d["spec"]), qkv, d["cache_k"].data_ptr(), d["cache_v"].data_ptr(), pm,
+                                                   dec.operand, g["k2"], T, 0)))
+    out.append(_entry("prefill: attention, window %d" % WINDOW, us, flops=_attn_flops(T, s["heads"], s["head_dim"], WINDOW)))
+    us = sweep(lambda d: ck(L.dh_attn_spec_kv_write(ctypes.byref(d["spec"]), qkv, d["cache_k"].data_ptr(), d["cache_v"].data_ptr(), T, 0)))
+    out.append(_entry("prefill: value norm + KV write", us, nbytes=6.0 * T * s["kv_heads"] * (g["D"] + g["VD"])))
+    t.close()
+    return out
+
+
+def q4k_kernels(dec, s, T):
+    from . import capi, synth
+    L, ck, c = dec.L, capi.check, dec.cfg
+    t, pos = _Timer(L), PROMPT + 8
+    Hd, I, H, Hkv, D = c["hidden"], c["inter"], c["heads"], c["kv_heads"], c["head_dim"]
+    qkv_n, b = dec.qs + 2 * dec.ks, dec._pf
+    out = []
+    sweep = lambda f: t.us([(lambda d=d: f(d)) for d in dec.layers])
+    for rows, x, normed, qkv, attn, act, y in ((1, dec.x, dec.normed, dec.qkv, dec.attn, dec.act, dec.x2),
+                                               (T, b["x"], b["normed"], b["qkv"], b["attn"], b["act"], b["x2"])):
+        def add(name, us, n, k, mats=1):
+            phase = "decode: " if rows == 1 else "prefill: "
+            out.append(_entry(phase + name, us, nbytes=float(mats * synth.q4k_nbytes(n, k))) if rows == 1 else
+                       _entry(phase + name, us, flops=2.0 * rows * n * k * mats))
+        add("norm + q/k/v", sweep(lambda d: ck(L.dh_q4k_matmul_rmsnorm(x.data_ptr(), d["input_norm"].data_ptr(), c["eps"], 0, d["wqkv"].data_ptr(),
+                                                                       qkv.data_ptr(), capi.F32, rows, qkv_n, Hd, 1.0, None))), qkv_n, Hd)
+        add("o + residual", sweep(lambda d: ck(L.dh_q4k_matmul(attn.data_ptr(), capi.F32, d["wo"].data_ptr(), y.data_ptr(), capi.F32, rows, Hd,
+                                                               dec.qs, 1.0, x.data_ptr()))), Hd, dec.qs)
+        add("norm + gate/up", sweep(lambda d: ck(L.dh_q4k_ffn_gate_up_rmsnorm(
+            x.data_ptr(), d["post_attn_norm"].data_ptr(), c["eps"], 0, d["wgate"].data_ptr(), d["wup"].data_ptr(), act.data_ptr(), rows, Hd, I,
+            capi.ACT_SILU, 1.0, 0.0))), I, Hd, 2)
+        add("down + residual", sweep(lambda d: ck(L.dh_q4k_matmul(act.data_ptr(), capi.F32, d["wdown"].data_ptr(), y.data_ptr(), capi.F32, rows,
+                                                                  Hd, I, 1.0, x.data_ptr()))), Hd, I)
+    us = sweep(lambda d: ck(L.dh_attn_decode_qkv(dec.qkv.data_ptr(), d["q_norm"].data_ptr(), d["k_norm"].data_ptr(), dec.cos.data_ptr(),
+                                                 dec.sin.data_ptr(), d["cache_k"].data_ptr(), d["cache_v"].data_ptr(), dec.attn.data_ptr(), H, Hkv,
+                                                 D, pos, D, 0, c["eps"], 0, 1, dec.scale, 0.0, WINDOW, 0, capi.KV_CONTIGUOUS, dec.attn_ws.data_ptr())))
+    out.append(_entry("decode: attention, %d keys" % WINDOW, us, nbytes=4.0 * WINDOW * Hkv * D))
+    us = sweep(lambda d: dec._enqueue_head(dec.x.data_ptr(), 0, None))
+    out.append(_entry("decode: norm + head + argmax (weights in cache where they fit)", us, nbytes=2.0 * c["vocab"] * Hd))
+    us = sweep(lambda d: ck(L.dh_attn_prefill(b["q"].data_ptr(), d["cache_k"].data_ptr(), d["cache_v"].data_ptr(), b["attn"].data_ptr(), T, H, Hkv,
+                                              D, T, dec.scale, 1, 0, 0.0, WINDOW)))
+    out.append(_entry("prefill: attention, window %d" % WINDOW, us, flops=_attn_flops(T, H, D, WINDOW)))
+    us = sweep(lambda d: ck(L.dh_qkv_norm_rope_kvwrite(b["qkv"].data_ptr(), d["q_norm"].data_ptr(), d["k_norm"].data_ptr(), dec.cos.data_ptr(),
+                                                       dec.sin.data_ptr(), b["q"].data_ptr(), d["cache_k"].data_ptr(), d["cache_v"].data_ptr(), T, H,
+                                                       Hkv, D, 0, D, 0, c["eps"], 0, 0, 1)))
+    out.append(_entry("prefill: q/k norm + RoPE + KV write", us, nbytes=float(T * D * (8 * H + 6 * 2 * Hkv))))
+    t.close()
+    return out
+
+
+def run(sizes, steps, warmup):
+    from . import decoder, dense_decoder
+    results = {}
+    for name in sizes:
+        s = SIZES[name]
+        max_seq = PROMPT + warmup + steps + 80
+        prompt = np.random.Generator(np.random.PCG64(1)).integers(0, VOCAB, PROMPT)
+        r = dict(s, vocab=VOCAB, window=WINDOW, prompt=PROMPT)
+        cfg = zepavik_config(s, max_seq)
+        dec = dense_decoder.DenseDecoder(cfg, dense_decoder.random_weights(cfg, seed=2), max_seq)
+        pre, step = _throughput(dec, prompt, steps, warmup)
+        nbytes = dec.weight_bytes_per_token(PROMPT + steps // 2)
+        r["zepavik"] = dict(prefill_tokens_per_s=round(pre, 1), decode_tokens_per_s=round(step, 1),
+                            decode_hbm_frac=round(nbytes * step / 1e9 / HBM_GBPS, 4), kernels=zepavik_kernels(dec, s, PROMPT))
+        log("[bench] zepavik %s: prefill %.0f tok/s, decode %.1f tok/s" % (name, pre, step))
+        del dec
+        cfg = q4k_config(s, max_seq)
+        layers, embed, final_norm, cos, sin = decoder.random_model(cfg, seed=3, max_seq=max_seq)
+        dec = decoder.HipDecoder(cfg, layers, embed, final_norm, cos, sin, max_seq)
+        pre, step = _throughput(dec, prompt, steps, warmup)
+        nbytes = dec.weight_bytes_per_token(PROMPT + steps // 2)
+        r["q4k"] = dict(prefill_tokens_per_s=round(pre, 1), decode_tokens_per_s=round(step, 1),
+                        decode_hbm_frac=round(nbytes * step / 1e9 / HBM_GBPS, 4), kernels=q4k_kernels(dec, s, PROMPT))
+        log("[bench] q4k %s: prefill %.0f tok/s, decode %.1f tok/s" % (name, pre, step))
+        del dec
+        results[name] = r
+    return results
