@@ -62,7 +62,9 @@ def build_hip(jobs=4, srcs=None, lib=LIB):
     with ThreadPoolExecutor(max_workers=jobs) as ex:
         list(ex.map(lambda so: _run([HIPCC] + HIP_FLAGS + FILE_FLAGS.get(os.path.basename(so[0]), []) +
                                     ["-c", so[0], "-o", so[1]]), zip(srcs, objs)))
-    _run([HIPCC, "--offload-arch=gfx950", "-shared", "-fPIC", "-o", lib] + objs)
+    # linked beside its place and moved there: an interrupted build leaves no half-written library behind
+    _run([HIPCC, "--offload-arch=gfx950", "-shared", "-fPIC", "-o", lib + ".part"] + objs)
+    os.replace(lib + ".part", lib)
     return lib
 
 

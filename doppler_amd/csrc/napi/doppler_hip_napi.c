@@ -397,6 +397,65 @@ FN(js_check_finiteness) {
   return ret_rc(env, dh_check_finiteness(in, dt, n, (uint32_t*)st, (uint32_t)layer, (uint32_t)step, thr));
 }
 
+/* ---- dense bf16 weights; the attention spec travels as bytes (size checked here) ---- */
+FN(js_dense_matmul) {
+  ARGS(18); P(0, A); I(1, adt); I(2, lda); P(3, W); I(4, ldw); I(5, M); I(6, N); I(7, K); F(8, alpha); P(9, bias); P(10, res);
+  P(11, C); I(12, ldc); I(13, first); P(14, C2); I(15, c2dt); I(16, ldc2); I(17, act);
+  return ret_rc(env, dh_dense_matmul(A, adt, lda, W, ldw, M, N, K, alpha, (const float*)bias, (const float*)res, (float*)C, ldc,
+                                     first, C2, c2dt, ldc2, act));
+}
+FN(js_dense_gemv) {
+  ARGS(15); P(0, x); P(1, nw); I(2, hid); F(3, eps); P(4, W); I(5, ldw); I(6, N); I(7, K); F(8, alpha); P(9, bias); P(10, res);
+  P(11, C); I(12, first); P(13, C2); I(14, act);
+  return ret_rc(env, dh_dense_gemv((const float*)x, (const float*)nw, hid, eps, W, ldw, N, K, alpha, (const float*)bias,
+                                   (const float*)res, (float*)C, first, (float*)C2, act));
+}
+FN(js_dense_lmhead_argmax) {
+  ARGS(13); P(0, x); P(1, nw); I(2, hid); F(3, eps); P(4, W); I(5, ldw); I(6, vocab); I(7, K); F(8, alpha); P(9, ws); P(10, tok);
+  I(11, idx); P(12, logits);
+  return ret_rc(env, dh_dense_lmhead_argmax((const float*)x, (const float*)nw, hid, eps, W, ldw, vocab, K, alpha, ws,
+                                            (uint32_t*)tok, idx, (float*)logits));
+}
+FN(js_embed_sum) {
+  ARGS(17); P(0, ids); I(1, off); P(2, prev); P(3, e); I(4, vocab); P(5, b); L(6, buckets); L(7, mp); L(8, mc); P(9, pos);
+  I(10, maxPos); P(11, out); I(12, ld); I(13, T); I(14, hid); I(15, start); P(16, kvLen);
+  return ret_rc(env, dh_embed_sum((const uint32_t*)ids, off, (const uint32_t*)prev, e, vocab, b, buckets, mp, mc, pos, maxPos,
+                                  (float*)out, ld, T, hid, start, (const uint32_t*)kvLen));
+}
+FN(js_rmsnorm_rows) {
+  ARGS(10); P(0, x); I(1, ldx); P(2, rows); P(3, w); P(4, out); I(5, dt); I(6, ldo); I(7, n); I(8, hid); F(9, eps);
+  return ret_rc(env, dh_rmsnorm_rows((const float*)x, ldx, (const uint32_t*)rows, (const float*)w, out, dt, ldo, n, hid, eps));
+}
+FN(js_attn_spec_bytes) { (void)info; return ret_num(env, (double)sizeof(dh_attn_spec)); }
+FN(js_attn_spec_workspace_bytes) { ARGS(3); I(0, H); I(1, VD); I(2, kv); return ret_num(env, (double)dh_attn_spec_workspace_bytes(H, VD, kv)); }
+static const dh_attn_spec* arg_spec(napi_env env, napi_value v) {
+  void* data = NULL; size_t len = 0;
+  if (!arg_bytes(env, v, &data, &len)) return NULL;
+  if (len < sizeof(dh_attn_spec)) {
+    napi_throw_error(env, NULL, "[attnSpec] the spec bytes are shorter than the struct");
+    return NULL;
+  }
+  return (const dh_attn_spec*)data;
+}
+FN(js_attn_spec_kv_write) {
+  ARGS(6); P(1, qkv); P(2, ck); P(3, cv); I(4, T); I(5, start);
+  const dh_attn_spec* s = arg_spec(env, a[0]);
+  if (!s) return NULL;
+  return ret_rc(env, dh_attn_spec_kv_write(s, (const float*)qkv, ck, cv, T, start));
+}
+FN(js_attn_spec_prefill) {
+  ARGS(9); P(1, qkv); P(2, ck); P(3, cv); P(4, out); I(5, dt); I(6, ld); I(7, T); I(8, start);
+  const dh_attn_spec* s = arg_spec(env, a[0]);
+  if (!s) return NULL;
+  return ret_rc(env, dh_attn_spec_prefill(s, (const float*)qkv, ck, cv, out, dt, ld, T, start));
+}
+FN(js_attn_spec_decode) {
+  ARGS(9); P(1, qkv); P(2, ck); P(3, cv); P(4, out); I(5, pos); P(6, kvLen); I(7, maxKvLen); P(8, ws);
+  const dh_attn_spec* s = arg_spec(env, a[0]);
+  if (!s) return NULL;
+  return ret_rc(env, dh_attn_spec_decode(s, (const float*)qkv, ck, cv, (float*)out, pos, (const uint32_t*)kvLen, maxKvLen, ws));
+}
+
 static napi_value module_init(napi_env env, napi_value exports) {
   static const struct { const char* name; napi_callback fn; } table[] = {
       {"graphBegin", js_graph_begin}, {"graphEnd", js_graph_end}, {"graphLaunch", js_graph_launch}, {"graphSetMaxPosition", js_graph_set_max_position}, {"graphPrepare", js_graph_prepare},
@@ -427,6 +486,10 @@ static napi_value module_init(napi_env env, napi_value exports) {
       {"sampleTopkWorkspaceBytes", js_sample_topk_workspace_bytes}, {"sampleTopk", js_sample_topk},
       {"castF32ToF16", js_cast_f32_to_f16}, {"castF16ToF32", js_cast_f16_to_f32},
       {"matmulRmsnormF32", js_matmul_rmsnorm_f32}, {"matmulRmsnormF16", js_matmul_rmsnorm_f16}, {"checkFiniteness", js_check_finiteness},
+      {"denseMatmul", js_dense_matmul}, {"denseGemv", js_dense_gemv}, {"denseLmheadArgmax", js_dense_lmhead_argmax},
+      {"embedSum", js_embed_sum}, {"rmsnormRows", js_rmsnorm_rows}, {"attnSpecBytes", js_attn_spec_bytes},
+      {"attnSpecWorkspaceBytes", js_attn_spec_workspace_bytes}, {"attnSpecKvWrite", js_attn_spec_kv_write},
+      {"attnSpecPrefill", js_attn_spec_prefill}, {"attnSpecDecode", js_attn_spec_decode},
   };
   for (size_t i = 0; i < sizeof(table) / sizeof(table[0]); i++) {
     napi_value fn;

@@ -9,6 +9,10 @@ export {
   recordLayerChain, recordDecodeAttentionPartials, layerChainSupported, layerChainMergesAttention, packChainPhases,
   packChainAttnSource,
 } from './gemv-chain.js';
+export {
+  recordEmbedSum, recordRMSNormRows, recordDenseMatmul, recordDenseGemv, recordDenseLmHeadArgmax, packAttnSpec,
+  recordAttnSpecKVWrite, recordAttnSpecPrefill, recordAttnSpecDecode,
+} from './dense.js';
 export { runRMSNorm, recordRMSNorm } from './rmsnorm.js';
 export { runRMSNormQK, recordRMSNormQK, canUseRMSNormQK } from './rmsnorm-qk.js';
 export {

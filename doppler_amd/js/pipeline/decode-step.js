@@ -1,52 +1,26 @@
-// Greedy decode loop over the HIP op API: the shape of the reference's decodeStep
-// (src/inference/pipelines/text/generator-steps.js:588-820) for a Qwen3-class Q4_K model.
-// One CommandRecorder per token, every op recorded in execution-graph order
-// (src/config/conversion/qwen3/qwen-3-embedding-0-6b-q4k-ehf16-af32.json `execution.decode`),
-// one 4-byte readback per token.
+// The Qwen3-class Q4_K model over the HIP op API: the ops of the reference's decodeStep
+// (src/inference/pipelines/text/generator-steps.js:588-820), recorded in execution-graph order
+// (src/config/conversion/qwen3/qwen-3-embedding-0-6b-q4k-ehf16-af32.json `execution.decode`).
+// The loops around them are TextDecoder's.
 import {
-  createTensor, createWeightBuffer, acquireBuffer, releaseBuffer, uploadData, readBufferSlice,
-  createCommandRecorder, recordGather, recordRMSNorm, recordMatmul, recordSplitQKVRMSNormRoPEQK,
-  recordAttention, recordFusedNormedFFN, recordFusedFFN, recordLmHeadArgmaxF16, lmHeadArgmaxNormFusable, recordGPUSample,
+  createTensor, createWeightBuffer, acquireBuffer, releaseBuffer,
+  recordGather, recordRMSNorm, recordMatmul, recordSplitQKVRMSNormRoPEQK,
+  recordAttention, recordFusedNormedFFN, recordFusedFFN, recordLmHeadArgmaxF16, lmHeadArgmaxNormFusable,
   recordDecodeAttentionFromQKV, decodeAttentionFromQKVSupported,
   recordLayerChain, recordDecodeAttentionPartials, layerChainSupported, layerChainMergesAttention,
-  recordCheckFiniteness, parseFinitenessStatusWords, resolveFinitenessAbsThreshold, FINITENESS_STATUS_BYTES,
+  recordCheckFiniteness,
 } from '../kernel-selector.js';
-import { getNative } from '../native.js';
+import { TextDecoder, FinitenessError, bufferWindow, upload } from './text-decoder.js';
 
-// A window of a device buffer starting `offset` bytes in (no ownership: never released).
-function bufferWindow(buffer, offset, size) {
-  return { ptr: buffer.ptr + BigInt(offset), size, capacity: size, label: buffer.label };
-}
+export { FinitenessError };
 
-// An activation left the f16 range (or the configured bound) during a decode step
-// (reference: src/inference/pipelines/text/generator-steps.js:164-169).
-export class FinitenessError extends Error {
-  constructor(message) {
-    super(message);
-    this.name = 'FinitenessError';
-  }
-}
-
-function upload(bytes, label) {
-  const buf = acquireBuffer(bytes.byteLength, undefined, label);
-  uploadData(buf, bytes);
-  return buf;
-}
-
-// decodeGreedy: tokens in flight between the device and the host (ring slots), and the events that mark
-// their copies
-const TOKEN_RING = 64;
-const READ_EVENTS = 4;
-
-export class HipTextDecoder {
+export class HipTextDecoder extends TextDecoder {
   // config: {layers, hidden, inter, heads, kvHeads, headDim, vocab, eps, maxSeq}
-  //   finitenessGuard (default false): check every layer's output against finitenessAbsThreshold
-  //   (one more launch per layer) and read the status words back beside the token, as the
-  //   reference does for f16 activations (layer.js:1237-1252, generator-steps.js:786-798, :837-843)
+  //   finitenessGuard, finitenessAbsThreshold: see TextDecoder
   // weights: {layers: [{wqkv, wo, wgate, wup, wdown (Uint8Array Q4_K), inputNorm, postAttnNorm,
   //           qNorm, kNorm (Float32Array)}], embed (Uint16Array f16 bits), finalNorm, cos, sin}
   constructor(config, weights) {
-    this.config = config;
+    super(config);
     const c = config;
     this.qSize = c.heads * c.headDim;
     this.kSize = c.kvHeads * c.headDim;
@@ -75,14 +49,10 @@ export class HipTextDecoder {
     // attention's key splits (two launches per layer), where the shapes are served and the guard is off
     this.chainGemvs = config.chainGemvs !== false && this.fuseQkvAttention && config.finitenessGuard !== true &&
       layerChainSupported(c.hidden, c.inter, this.qSize) && layerChainMergesAttention(c.heads, c.kvHeads, c.headDim, c.maxSeq);
-    this.ids = acquireBuffer(16, undefined, 'token_ids');
-    // [token, status, layer, step, pad]: the staging layout of the reference's guarded readback
-    this.tokenOut = acquireBuffer(4 + FINITENESS_STATUS_BYTES, undefined, 'sampled_token');
-    this.finitenessGuard = config.finitenessGuard === true;
-    this.finitenessAbsThreshold = resolveFinitenessAbsThreshold(config.finitenessAbsThreshold);
-    this.finitenessStatus = bufferWindow(this.tokenOut, 4, FINITENESS_STATUS_BYTES);
-    this.logits = null;
-    this.readback = null;
+  }
+
+  deviceKvLenServed() {
+    return this.fuseQkvAttention;
   }
 
   // Final RMSNorm + LM head + argmax of one hidden row: one launch with the norm inside the LM head kernel
@@ -99,118 +69,65 @@ export class HipTextDecoder {
     await recordLmHeadArgmaxF16(recorder, normed, this.embed, opts);
   }
 
-  // Final RMSNorm + LM head for one hidden row; greedy, or top-k temperature sampling when
-  // `sampling` = {temperature, topK, randomSeed} is given (the logits then go through memory).
-  async recordHead(recorder, temps, hiddenRow, sampling, tokenOut = this.tokenOut, tokenIndex = 0) {
-    const c = this.config;
-    if (sampling && !this.logits) this.logits = acquireBuffer(c.vocab * 4, undefined, 'logits');
-    await this.recordNormedLmHead(recorder, temps, hiddenRow, tokenOut, tokenIndex, sampling ? this.logits : null);
-    if (sampling) {
-      await recordGPUSample(recorder, this.logits, c.vocab, Object.assign({ outputBuffer: tokenOut, outputIndex: tokenIndex }, sampling));
-    }
-  }
-
-  // Pushes prompt tokens through the batched path (prefill GEMMs + prefill attention), `chunk`
-  // tokens per pass, writing KV rows startPos.. ; returns the token after the last prompt token.
-  // Mirrors the reference's prefill (src/inference/pipelines/text/generator.js) on the HIP ops.
-  async prefill(tokens, startPos = 0, options = {}) {
-    const c = this.config;
-    const chunk = Math.max(1, Math.min(options.chunk || 2048, tokens.length));
-    if (tokens.length === 0 || startPos + tokens.length > c.maxSeq) {
-      throw new Error(`[prefill] ${tokens.length} tokens at ${startPos} do not fit maxSeq=${c.maxSeq}`);
-    }
-    const recorder = createCommandRecorder('prefill');
-    const temps = [];
+  // A portion through the batched path: prefill GEMMs + prefill attention.
+  async recordPrefillChunk(recorder, temps, ids, part, pos) {
+    const c = this.config, T = part.length;
     const temp = (t) => { temps.push(t.buffer); return t; };
-    const ids = acquireBuffer(chunk * 4, undefined, 'prefill_ids');
-    temps.push(ids);
-    let x = null, T = 0;
-    for (let c0 = 0; c0 < tokens.length; c0 += chunk) {
-      const part = tokens.slice(c0, c0 + chunk);
-      T = part.length;
-      const pos = startPos + c0;
-      uploadData(ids, new Uint32Array(part));
-      x = temp(await recordGather(recorder, ids, this.embed, T, c.hidden, c.vocab, { embeddingDtype: 'f16', outputDtype: 'f32' }));
-      for (let li = 0; li < this.layers.length; li++) {
-        const l = this.layers[li];
-        // the input RMSNorm runs inside the product (GEMV prologue below 16 tokens, the GEMM's activation
-        // packing from 16 on) unless the model asks for separate norm launches
-        const fusedNorm = c.fuseNorm !== false;
-        let qkv;
-        if (fusedNorm) {
-          qkv = temp(await recordMatmul(recorder, x, l.wqkv, T, this.qSize + 2 * this.kSize, c.hidden,
-            { outputDtype: 'f32', role: 'qkv_proj', layerIdx: li,
-              normWeight: l.inputNorm, rmsNormEps: c.eps, useFusedRmsnormWideTile: true }));
-        } else {
-          const normed = temp(await recordRMSNorm(recorder, x, l.inputNorm, c.eps, { batchSize: T, hiddenSize: c.hidden }));
-          qkv = temp(await recordMatmul(recorder, normed, l.wqkv, T, this.qSize + 2 * this.kSize, c.hidden,
-            { outputDtype: 'f32', role: 'qkv_proj', layerIdx: li }));
-        }
-        const split = await recordSplitQKVRMSNormRoPEQK(recorder, qkv, l.qNorm, l.kNorm, this.cos, this.sin, c.eps, {
-          numTokens: T, numHeads: c.heads, numKVHeads: c.kvHeads, headDim: c.headDim,
-          qSize: this.qSize, kSize: this.kSize, vSize: this.kSize, startPos: pos,
-          f16KVCacheWrite: { keysBuffer: l.cacheK.buffer, valuesBuffer: l.cacheV.buffer, dstOffset: pos * this.kSize },
-        });
-        temp(split.Q);
-        const attn = temp(await recordAttention(recorder, split.Q, l.cacheK, l.cacheV, null, c.heads, c.headDim, {
-          seqLen: T, kvLen: pos + T, numKVHeads: c.kvHeads, causal: true, startPos: pos, layerIdx: li,
-        }));
-        const attnFlat = createTensor(attn.buffer, 'f32', [T, this.qSize], 'attn_flat');
-        const x2 = temp(await recordMatmul(recorder, attnFlat, l.wo, T, c.hidden, this.qSize,
-          { outputDtype: 'f32', role: 'o_proj', layerIdx: li, residualTensor: x }));
-        let act;
-        if (fusedNorm) {
-          act = temp(await recordFusedNormedFFN(recorder, x2, l.postAttnNorm, c.eps, l.wgate, l.wup, c.hidden, c.inter,
-            { batchSize: T, activation: 'silu' }));
-        } else {
-          const normed2 = temp(await recordRMSNorm(recorder, x2, l.postAttnNorm, c.eps, { batchSize: T, hiddenSize: c.hidden }));
-          act = temp(await recordFusedFFN(recorder, normed2, l.wgate, l.wup, c.hidden, c.inter,
-            { batchSize: T, activation: 'silu' }));
-        }
-        x = temp(await recordMatmul(recorder, act, l.wdown, T, c.hidden, c.inter,
-          { outputDtype: 'f32', role: 'down_proj', layerIdx: li, residualTensor: x2 }));
+    let x = temp(await recordGather(recorder, bufferWindow(ids, 4, 4 * T), this.embed, T, c.hidden, c.vocab, { embeddingDtype: 'f16', outputDtype: 'f32' }));
+    for (let li = 0; li < this.layers.length; li++) {
+      const l = this.layers[li];
+      // the input RMSNorm runs inside the product (GEMV prologue below 16 tokens, the GEMM's activation
+      // packing from 16 on) unless the model asks for separate norm launches
+      const fusedNorm = c.fuseNorm !== false;
+      let qkv;
+      if (fusedNorm) {
+        qkv = temp(await recordMatmul(recorder, x, l.wqkv, T, this.qSize + 2 * this.kSize, c.hidden,
+          { outputDtype: 'f32', role: 'qkv_proj', layerIdx: li,
+            normWeight: l.inputNorm, rmsNormEps: c.eps, useFusedRmsnormWideTile: true }));
+      } else {
+        const normed = temp(await recordRMSNorm(recorder, x, l.inputNorm, c.eps, { batchSize: T, hiddenSize: c.hidden }));
+        qkv = temp(await recordMatmul(recorder, normed, l.wqkv, T, this.qSize + 2 * this.kSize, c.hidden,
+          { outputDtype: 'f32', role: 'qkv_proj', layerIdx: li }));
       }
+      const split = await recordSplitQKVRMSNormRoPEQK(recorder, qkv, l.qNorm, l.kNorm, this.cos, this.sin, c.eps, {
+        numTokens: T, numHeads: c.heads, numKVHeads: c.kvHeads, headDim: c.headDim,
+        qSize: this.qSize, kSize: this.kSize, vSize: this.kSize, startPos: pos,
+        f16KVCacheWrite: { keysBuffer: l.cacheK.buffer, valuesBuffer: l.cacheV.buffer, dstOffset: pos * this.kSize },
+      });
+      temp(split.Q);
+      const attn = temp(await recordAttention(recorder, split.Q, l.cacheK, l.cacheV, null, c.heads, c.headDim, {
+        seqLen: T, kvLen: pos + T, numKVHeads: c.kvHeads, causal: true, startPos: pos, layerIdx: li,
+      }));
+      const attnFlat = createTensor(attn.buffer, 'f32', [T, this.qSize], 'attn_flat');
+      const x2 = temp(await recordMatmul(recorder, attnFlat, l.wo, T, c.hidden, this.qSize,
+        { outputDtype: 'f32', role: 'o_proj', layerIdx: li, residualTensor: x }));
+      let act;
+      if (fusedNorm) {
+        act = temp(await recordFusedNormedFFN(recorder, x2, l.postAttnNorm, c.eps, l.wgate, l.wup, c.hidden, c.inter,
+          { batchSize: T, activation: 'silu' }));
+      } else {
+        const normed2 = temp(await recordRMSNorm(recorder, x2, l.postAttnNorm, c.eps, { batchSize: T, hiddenSize: c.hidden }));
+        act = temp(await recordFusedFFN(recorder, normed2, l.wgate, l.wup, c.hidden, c.inter,
+          { batchSize: T, activation: 'silu' }));
+      }
+      x = temp(await recordMatmul(recorder, act, l.wdown, T, c.hidden, c.inter,
+        { outputDtype: 'f32', role: 'down_proj', layerIdx: li, residualTensor: x2 }));
     }
-    const lastRow = createTensor(bufferWindow(x.buffer, (T - 1) * c.hidden * 4, c.hidden * 4), 'f32', [1, c.hidden], 'last_hidden');
-    await this.recordHead(recorder, temps, lastRow, options.sampling || null);
-    for (const b of temps) recorder.trackTemporaryBuffer(b);
-    recorder.submit();
-    const bytes = await readBufferSlice(this.tokenOut, 0, 4);
-    return new Uint32Array(bytes)[0];
+    return { buffer: x.buffer, rowFloats: c.hidden };
   }
 
-  // prefill + decode loop: returns the generated token ids.  sampling = {temperature, topK, seed}
-  // draws token i with randomSeed seed + i (greedy when absent), as the reference's generator
-  // advances its seed per step.
-  async generate(promptTokens, maxTokens, sampling = null) {
-    const draw = (i) => (sampling ? { temperature: sampling.temperature, topK: sampling.topK, randomSeed: sampling.seed + i } : null);
-    const out = [];
-    let tok = await this.prefill(promptTokens, 0, { sampling: draw(0) });
-    out.push(tok);
-    for (let i = 1; i < maxTokens; i++) {
-      tok = await this.decodeStep(tok, promptTokens.length + i - 1, { sampling: draw(i) });
-      out.push(tok);
-    }
-    return out;
-  }
-
-  // Records the ops of one decode step for the token id in this.ids at position `pos`; the new
-  // token id goes to this.tokenOut.  Temporaries are pushed onto `temps`.
-  // options.idsBuffer: the input token id is read from this device word instead; options.tokenOutBuffer /
-  // tokenOutIndex: the new token goes to that word of that buffer instead.
-  async recordDecodeStep(recorder, temps, pos, options = {}) {
+  async recordEmbedding(recorder, temps, ids, prev, pos, options) {
     const c = this.config;
-    if (!(pos >= 0 && pos < c.maxSeq)) {
-      // the ops take no cache capacity: a position past the caches would write K/V out of bounds
-      throw new Error(`[decodeStep] position ${pos} is outside the KV cache (maxSeq=${c.maxSeq})`);
-    }
+    const x = await recordGather(recorder, ids, this.embed, 1, c.hidden, c.vocab, { embeddingDtype: 'f16', outputDtype: 'f32' });
+    temps.push(x.buffer);
+    return x;
+  }
+
+  async recordLayers(recorder, temps, x, pos, options) {
+    const c = this.config;
     const temp = (t) => { temps.push(t.buffer); return t; };
-    const tokenOut = options.tokenOutBuffer || this.tokenOut, tokenIndex = options.tokenOutIndex || 0;
-    let x = temp(await recordGather(recorder, options.idsBuffer || this.ids, this.embed, 1, c.hidden, c.vocab,
-      { embeddingDtype: 'f16', outputDtype: 'f32' }));
-    if (this.chainGemvs) {
-      x = await this.recordChainedLayers(recorder, temps, x, pos, options);
-    } else for (let li = 0; li < this.layers.length; li++) {
+    if (this.chainGemvs) return this.recordChainedLayers(recorder, temps, x, pos, options);
+    for (let li = 0; li < this.layers.length; li++) {
       const l = this.layers[li];
       // input RMSNorm runs in the prologue of the stacked q/k/v projection
       const qkv = temp(await recordMatmul(recorder, x, l.wqkv, 1, this.qSize + 2 * this.kSize, c.hidden,
@@ -244,11 +161,7 @@ export class HipTextDecoder {
         recordCheckFiniteness(recorder, x, c.hidden, this.finitenessStatus, li, pos, this.finitenessAbsThreshold);
       }
     }
-    if (options.sampling) {
-      await this.recordHead(recorder, temps, x, options.sampling, tokenOut, tokenIndex);
-    } else {
-      await this.recordNormedLmHead(recorder, temps, x, tokenOut, tokenIndex, options.logitsOutput || null);
-    }
+    return x;
   }
 
   // The layers of a decode step at two launches each: the attention's split kernel, then one chained
@@ -289,147 +202,7 @@ export class HipTextDecoder {
     return createTensor(xb, 'f32', [1, c.hidden], 'layer_output');
   }
 
-  // Returns the greedy token for `token` at position `pos` (KV rows 0..pos-1 present).
-  // options.recorder: a recorder of the caller's (e.g. a profiling one) instead of a fresh one.
-  async decodeStep(token, pos, options = {}) {
-    const recorder = options.recorder || createCommandRecorder('decode');
-    const temps = [];
-    uploadData(this.ids, new Uint32Array([token]));
-    if (this.finitenessGuard) getNative().fillZero(this.tokenOut.ptr, 4, FINITENESS_STATUS_BYTES);
-    await this.recordDecodeStep(recorder, temps, pos, options);
-    for (const b of temps) recorder.trackTemporaryBuffer(b);
-    recorder.submit();
-    // the only device->host crossing: the token, with the guard's status words beside it
-    const bytes = await readBufferSlice(this.tokenOut, 0, this.finitenessGuard ? 4 + FINITENESS_STATUS_BYTES : 4);
-    const words = new Uint32Array(bytes);
-    if (this.finitenessGuard) {
-      const status = parseFinitenessStatusWords(words, 1);
-      if (status.triggered) throw new FinitenessError(`F16 bounds exceeded during generation${status.metadata}`);
-    }
-    return words[0];
-  }
-
-  // n greedy steps starting with `token` at position `pos`; returns the n new token ids.  Every step's
-  // token is read back (4 bytes per step, as in decodeStep), but one step late: step k + 1 takes its input
-  // token from device memory and is enqueued before the host waits for token k, whose copy into pinned
-  // memory was enqueued behind step k, so the GPU never waits for the host between steps (the reference
-  // stages its token readbacks through a ring the same way, src/inference/decode-ring.js:141-177).  A
-  // caller with a stop condition checks the tokens as they come and drops the one step in flight.
-  async decodeGreedy(token, pos, n) {
-    if (n <= 0) return [];
-    if (this.finitenessGuard) {
-      const guarded = [];
-      for (let k = 0; k < n; k++) {
-        token = await this.decodeStep(token, pos + k);
-        guarded.push(token);
-      }
-      return guarded;
-    }
-    const native = getNative();
-    if (!this.readback) {
-      const host = native.hostAlloc(4 * TOKEN_RING);
-      const events = [];
-      for (let i = 0; i < READ_EVENTS; i++) events.push(native.eventCreate());
-      this.readback = { host, tokens: new Uint32Array(host.view), events, ring: acquireBuffer(4 * TOKEN_RING, undefined, 'token_ring') };
-    }
-    const rb = this.readback;
-    const enqueueStep = async (k) => {
-      const recorder = createCommandRecorder('decode');
-      const temps = [];
-      const slot = k % TOKEN_RING;
-      const options = { tokenOutBuffer: rb.ring, tokenOutIndex: slot };
-      if (k > 0) options.idsBuffer = bufferWindow(rb.ring, 4 * ((k - 1) % TOKEN_RING), 4);
-      await this.recordDecodeStep(recorder, temps, pos + k, options);
-      for (const b of temps) recorder.trackTemporaryBuffer(b);
-      recorder.submit();
-      native.downloadAsync(rb.host.ptr, 4 * slot, rb.ring.ptr, 4 * slot, 4);
-      native.eventRecord(rb.events[k % READ_EVENTS]);
-    };
-    const waitToken = (k) => {
-      native.eventSynchronize(rb.events[k % READ_EVENTS]);
-      return rb.tokens[k % TOKEN_RING];
-    };
-    uploadData(this.ids, new Uint32Array([token]));
-    await enqueueStep(0);
-    const out = [];
-    for (let k = 1; k < n; k++) {
-      await enqueueStep(k);
-      out.push(waitToken(k - 1));
-    }
-    out.push(waitToken(n - 1));
-    return out;
-  }
-
-  // Frees the pinned staging memory, the device ring and the events decodeGreedy made.
-  releaseReadback() {
-    if (this.readback) {
-      const native = getNative();
-      native.sync();
-      for (const ev of this.readback.events) native.eventDestroy(ev);
-      this.readback.tokens = null;
-      native.hostFree(this.readback.host.ptr);
-      releaseBuffer(this.readback.ring);
-      this.readback = null;
-    }
-  }
-
-  // Captures the decode step into a HIP graph, the counterpart of the reference's
-  // one-submit-per-step recorder (generator-steps.js:605,814).  The step runs once normally first
-  // (every kernel's one-time set-up then lies outside the capture); the buffers the captured step
-  // uses stay allocated for the graph's life.
-  async captureDecodeStep(token, pos) {
-    if (!this.fuseQkvAttention) throw new Error('[captureDecodeStep] serves the fused-attention step');
-    const c = this.config;
-    const first = await this.decodeStep(token, pos);
-    uploadData(this.ids, new Uint32Array([token, pos + 1]));
-    getNative().graphBegin();
-    let graph = null;
-    const temps = [];
-    try {
-      // with the guard on the captured step also clears the status words (the library moves the
-      // checks' step number with the position at every replay)
-      if (this.finitenessGuard) getNative().fillZero(this.tokenOut.ptr, 4, FINITENESS_STATUS_BYTES);
-      await this.recordDecodeStep(createCommandRecorder('decode_capture'), temps, pos, { deviceKvLen: true });
-    } finally {
-      graph = getNative().graphEnd(pos);
-    }
-    getNative().graphSetMaxPosition(graph, c.maxSeq - 1);
-    this.graph = graph;
-    this.graphBuffers = temps;
-    return first;
-  }
-
-  // One decode step by replaying the captured graph at position `pos`.
-  async decodeStepGraph(token, pos) {
-    const c = this.config;
-    if (!(pos >= 0 && pos < c.maxSeq)) {
-      throw new Error(`[decodeStepGraph] position ${pos} is outside the KV cache (maxSeq=${c.maxSeq})`);
-    }
-    if (!this.graph) return this.captureDecodeStep(token, pos);
-    // token id and key count travel together; the attention kernels of the captured step read the count
-    uploadData(this.ids, new Uint32Array([token, pos + 1]));
-    getNative().graphLaunch(this.graph, pos);
-    const bytes = await readBufferSlice(this.tokenOut, 0, this.finitenessGuard ? 4 + FINITENESS_STATUS_BYTES : 4);
-    const words = new Uint32Array(bytes);
-    if (this.finitenessGuard) {
-      const status = parseFinitenessStatusWords(words, 1);
-      if (status.triggered) throw new FinitenessError(`F16 bounds exceeded during generation${status.metadata}`);
-    }
-    return words[0];
-  }
-
-  releaseGraph() {
-    if (this.graph) {
-      getNative().graphDestroy(this.graph);
-      for (const b of this.graphBuffers) releaseBuffer(b);
-      this.graph = null;
-      this.graphBuffers = [];
-    }
-  }
-
-  destroy() {
-    this.releaseGraph();
-    this.releaseReadback();
+  releaseWeights() {
     for (const l of this.layers) {
       for (const key of Object.keys(l)) releaseBuffer(l[key].buffer);
     }

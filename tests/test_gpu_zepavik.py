@@ -386,7 +386,7 @@ def test_bad_specs_are_refused(L):
 def folders(tmp_path_factory):
     base = tmp_path_factory.mktemp("zepavik")
     out = {}
-    for name, cfg, seed in (("mixed", zm.MIXED, 21), ("wide-heads", zm.WIDE_HEADS, 22), ("even", zm.EVEN, 23)):
+    for name, cfg, seed in (("mixed", zm.MIXED, 21), ("wide-heads", zm.WIDE_HEADS, 22), ("even", zm.EVEN, 23), ("odd", zm.ODD, 24)):
         t = zm.tensors(cfg, seed)
         out[name] = (zm.write(base / name, cfg, t), cfg, t)
     return out
@@ -404,7 +404,7 @@ def feed_all(dec, tokens, portions):
 
 
 @pytest.mark.parametrize("dtype,tol", [("float32", F32_ROW), ("bfloat16", BF16_ROW)])
-@pytest.mark.parametrize("name", ["mixed", "wide-heads", "even"])
+@pytest.mark.parametrize("name", ["mixed", "wide-heads", "even", "odd"])
 def test_logits_whole_decoded_and_in_portions(folders, name, dtype, tol):
     folder, cfg, t = folders[name]
     toks = zm.prompt(cfg, 180, 31)

@@ -57,7 +57,7 @@ def test_plain_model_is_causal_and_reads_the_previous_token():
 # ------------------------------------------------------------------ configuration, weights, registry
 
 def test_configuration_round_trip_and_unknown_keys_fail_closed():
-    for c in (zm.MIXED, zm.WIDE_HEADS, zm.EVEN):
+    for c in (zm.MIXED, zm.WIDE_HEADS, zm.EVEN, zm.ODD):
         assert zepavik.config_json(zepavik.decoder_config(c)) == c
 
     def broken(edit):
@@ -113,7 +113,7 @@ def test_truncated_files_are_refused(tmp_path):
         safetensors_file.SafetensorsFile(path)
 
 
-@pytest.mark.parametrize("cfg", [zm.MIXED, zm.WIDE_HEADS], ids=["mixed", "wide-heads"])
+@pytest.mark.parametrize("cfg", [zm.MIXED, zm.WIDE_HEADS, zm.ODD], ids=["mixed", "wide-heads", "odd"])
 def test_stacked_and_padded_weights_are_the_separate_products(tmp_path, cfg):
     t = zm.tensors(cfg, 7)
     c, w = zepavik.load_arrays(zm.write(tmp_path, cfg, t))

@@ -33,6 +33,8 @@ MIXED = config(136, 211, [layer(6, 2, 24, 40, 9, ff=88), layer(4, 4, 64, 32, 65,
                           layer(2, 1, 72, 104, 64, ff=56)], eps=3e-4, logit_scale=1.3)
 # many query heads per key/value head, heads wider than the matrix-core kernel's
 WIDE_HEADS = config(96, 130, [layer(12, 1, 16, 8, 40, ff=64), layer(3, 1, 136, 24, 70, ff=40), layer(2, 2, 40, 264, 21, ff=24)])
+# sizes that are multiples of nothing
+ODD = config(90, 131, [layer(3, 1, 7, 9, 5, ff=33), layer(2, 2, 33, 65, 17, scale=0.11, ff=1), layer(7, 7, 3, 5, 66)], buckets=1, eps=0.02)
 # even sizes, one kind of layer
 EVEN = config(192, 301, [layer(4, 2, 64, 64, 50, ff=256)] * 3)
 
