@@ -17,8 +17,10 @@ struct EmbedArgs {
   const uint32_t* kv_len;
 };
 
-// One workgroup per token.  Rows that do not exist (id or position out of range) count as zeros, so no id read on
+// Grid = (tokens, slices of 2048 columns): eight columns per thread with 16-byte loads where the rows are aligned for
+// them, else one column at a time.  Rows that do not exist (id or position out of range) count as zeros, so no id read on
 // the device can send a load outside the tables.
+template <bool VEC>
 __global__ __launch_bounds__(256) void embed_sum_kernel(const EmbedArgs a) {
   const int t = blockIdx.x;
   const int64_t p = a.kv_len ? (int64_t)*a.kv_len - 1 : (int64_t)a.start_pos + t;
@@ -36,7 +38,26 @@ __global__ __launch_bounds__(256) void embed_sum_kernel(const EmbedArgs a) {
   }
   const uint16_t* q = a.pos && p >= 0 && p < a.max_positions ? a.pos + p * a.hidden : nullptr;
   float* o = a.out + (int64_t)t * a.ld_out;
-  for (int i = threadIdx.x; i < a.hidden; i += 256) {
+  const int first = 2048 * blockIdx.y;
+  if (VEC) {
+    const int i = first + 8 * threadIdx.x;
+    if (i >= a.hidden) return;
+    const dh::u32x4_t none = {0u, 0u, 0u, 0u};
+    const dh::u32x4_t ev = e ? *reinterpret_cast<const dh::u32x4_t*>(e + i) : none;
+    const dh::u32x4_t bv = b ? *reinterpret_cast<const dh::u32x4_t*>(b + i) : none;
+    const dh::u32x4_t qv = q ? *reinterpret_cast<const dh::u32x4_t*>(q + i) : none;
+    float v[8];
+#pragma unroll
+    for (int w = 0; w < 4; w++) {
+      v[2 * w] = dh::bf16_low(ev[w]) + dh::bf16_low(bv[w]) + dh::bf16_low(qv[w]);
+      v[2 * w + 1] = dh::bf16_high(ev[w]) + dh::bf16_high(bv[w]) + dh::bf16_high(qv[w]);
+    }
+    reinterpret_cast<float4*>(o + i)[0] = make_float4(v[0], v[1], v[2], v[3]);
+    reinterpret_cast<float4*>(o + i)[1] = make_float4(v[4], v[5], v[6], v[7]);
+    return;
+  }
+  const int last = min(first + 2048, a.hidden);
+  for (int i = first + threadIdx.x; i < last; i += 256) {
     float v = e ? dh::bf16_bits_to_f32(e[i]) : 0.f;
     if (b) v += dh::bf16_bits_to_f32(b[i]);
     if (q) v += dh::bf16_bits_to_f32(q[i]);
@@ -123,7 +144,12 @@ int dh_embed_sum(const uint32_t* d_ids, int index_offset, const uint32_t* d_prev
   a.out = d_out; a.buckets = buckets; a.mul_prev = mul_prev; a.mul_cur = mul_cur;
   a.vocab = vocab; a.max_positions = max_positions; a.ld_out = ld_out; a.hidden = hidden; a.start_pos = start_pos;
   a.kv_len = d_kv_len;
-  hipLaunchKernelGGL(embed_sum_kernel, dim3(T), dim3(256), 0, dh::stream(), a);
+  const bool vec = hidden % 8 == 0 && ld_out % 4 == 0 &&
+                   ((reinterpret_cast<uintptr_t>(d_embed) | reinterpret_cast<uintptr_t>(d_bigram) | reinterpret_cast<uintptr_t>(d_pos) |
+                     reinterpret_cast<uintptr_t>(d_out)) & 15) == 0;
+  const dim3 grid((unsigned)T, (unsigned)dh::ceil_div(hidden, 2048));
+  if (vec) hipLaunchKernelGGL(embed_sum_kernel<true>, grid, dim3(256), 0, dh::stream(), a);
+  else hipLaunchKernelGGL(embed_sum_kernel<false>, grid, dim3(256), 0, dh::stream(), a);
   DH_CHECK_LAUNCH(op);
   return 0;
 }

@@ -121,6 +121,10 @@ def zepavik_kernels(dec, s, T):
     us = sweep(lambda d: ck(L.dh_dense_lmhead_argmax(dec.x.data_ptr(), dec.final_norm.data_ptr(), Hd, c["eps"], dec.head.data_ptr(),
                                                      dec.kx, c["vocab"], dec.kx, 1.0, dec.lm_ws.data_ptr(), dec.token.data_ptr(), 0, None)))
     out.append(_entry("decode: norm + head + argmax (weights in cache where they fit)", us, nbytes=2.0 * c["vocab"] * Hd))
+    us = t.us([lambda: dec._enqueue_embed(dec.ids.data_ptr(), dec.ids.data_ptr() + 8, pos, False)] * 20)
+    out.append(_entry("decode: embedding sum", us, nbytes=10.0 * Hd))
+    us = t.us([lambda: ck(L.dh_embed_sum(b["ids"].data_ptr(), 1, b["ids"].data_ptr(), *dec._embed_args(), x, dec.kx, T, Hd, 0, None))] * 10)
+    out.append(_entry("prefill: embedding sum", us, nbytes=10.0 * T * Hd))
     us = sweep(lambda d: dec._enqueue_in(d, x, b["normed"].data_ptr(), dec.operand, qkv, pm + elem * g["attn_cols"], T, g["k2"]))
     out.append(_entry("prefill: norm, q/k/v/gate/up", us, flops=2.0 * T * g["n"] * Hd))
     us = sweep(lambda d: dec._enqueue_out(d, pm, dec.operand, x, T))
@@ -161,6 +165,10 @@ def q4k_kernels(dec, s, T):
                                                  dec.sin.data_ptr(), d["cache_k"].data_ptr(), d["cache_v"].data_ptr(), dec.attn.data_ptr(), H, Hkv,
                                                  D, pos, D, 0, c["eps"], 0, 1, dec.scale, 0.0, WINDOW, 0, capi.KV_CONTIGUOUS, dec.attn_ws.data_ptr())))
     out.append(_entry("decode: attention, %d keys" % WINDOW, us, nbytes=4.0 * WINDOW * Hkv * D))
+    us = t.us([lambda: dec._enqueue_embed(dec.ids.data_ptr(), None, pos, False)] * 20)
+    out.append(_entry("decode: embedding gather", us, nbytes=6.0 * Hd))
+    us = t.us([lambda: ck(L.dh_gather_f16(b["ids"].data_ptr(), dec.embed.data_ptr(), b["x"].data_ptr(), T, Hd, c["vocab"], 0))] * 10)
+    out.append(_entry("prefill: embedding gather", us, nbytes=6.0 * T * Hd))
     us = sweep(lambda d: dec._enqueue_head(dec.x.data_ptr(), 0, None))
     out.append(_entry("decode: norm + head + argmax (weights in cache where they fit)", us, nbytes=2.0 * c["vocab"] * Hd))
     us = sweep(lambda d: ck(L.dh_attn_prefill(b["q"].data_ptr(), d["cache_k"].data_ptr(), d["cache_v"].data_ptr(), b["attn"].data_ptr(), T, H, Hkv,

@@ -48,7 +48,7 @@ def rng(seed):
 
 # ------------------------------------------------------------------ embedding, norms
 
-@pytest.mark.parametrize("hidden,buckets,mp,mc", [(136, 61, 31, 13), (70, 1, 5, 9), (256, 509, 2000003, 1999993)])
+@pytest.mark.parametrize("hidden,buckets,mp,mc", [(136, 61, 31, 13), (70, 1, 5, 9), (4104, 501, 2000003, 1999993), (2051, 77, 3, 2)])
 def test_embedding_sum(L, hidden, buckets, mp, mc):
     """Portions of a sequence; products of ids and multipliers far above 32 bits."""
     V, P, n = 3001, 90, 40
