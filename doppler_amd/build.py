@@ -43,9 +43,10 @@ def _run(cmd):
 
 
 # The families a model with dense weights runs on: the runtime, its glue ops, output heads and sampling, the dense
-# products and the attention they feed.
+# products, and the attentions, memories and experts they feed.
 DENSE_SOURCES = ("attention_prefill.hip", "attention_spec.hip", "dense_elementwise.hip", "dense_gemm.hip", "dense_gemv.hip",
-                 "dh_runtime.hip", "elementwise.hip", "lmhead.hip", "sample.hip")
+                 "dh_runtime.hip", "elementwise.hip", "experts.hip", "latent_attention.hip", "lmhead.hip", "matrix_memory.hip",
+                 "sample.hip")
 DENSE_LIB = os.path.join(LIB_DIR, "libdopplerhip_dense.so")
 
 

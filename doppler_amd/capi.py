@@ -12,7 +12,7 @@ LIB_PATH = os.path.join(_HERE, "lib", "libdopplerhip.so")
 DENSE_LIB_PATH = os.path.join(_HERE, "lib", "libdopplerhip_dense.so")
 
 F32, F16, BF16 = 0, 1, 2
-ACT_SILU, ACT_GELU, ACT_RELU2, ACT_NONE = 0, 1, 2, -1
+ACT_SILU, ACT_GELU, ACT_RELU2, ACT_GELU_ERF, ACT_NONE = 0, 1, 2, 3, -1
 KV_CONTIGUOUS, KV_RING = 0, 1
 PLAN_GEMV_I8, PLAN_GEMV_ROWS, PLAN_GEMV_RING, PLAN_GEMM, PLAN_GEMV_LDS = 1, 2, 3, 4, 5
 
@@ -45,6 +45,26 @@ class AttnSpec(ctypes.Structure):
     _fields_ = [("H", _I), ("Hkv", _I), ("D", _I), ("VD", _I), ("value_dim", _I), ("window", _I), ("cache_dtype", _I),
                 ("value_norm", _I), ("k_offset", _I), ("v_offset", _I), ("gate_offset", _I), ("ld_qkv", _I),
                 ("scale", _F), ("value_eps", _F), ("d_bias_r1", _P), ("d_bias_r2", _P)]
+
+
+class Latent(ctypes.Structure):
+    """struct dh_latent: one layer's attention over a low-rank latent."""
+    _fields_ = [("H", _I), ("D", _I), ("R", _I), ("VD", _I), ("rank", _I), ("C", _I), ("rot_dim", _I), ("window", _I),
+                ("cache_dtype", _I), ("dkv_offset", _I), ("ld_row", _I), ("scale", _F), ("eps", _F), ("d_latent_norm", _P), ("d_cos", _P),
+                ("d_sin", _P), ("d_uk", _P), ("d_uv", _P), ("d_uk_t", _P), ("d_uv_rows", _P)]
+
+
+class MLSTM(ctypes.Structure):
+    """struct dh_mlstm: one layer's matrix memory."""
+    _fields_ = [("H", _I), ("dim", _I), ("vdim", _I), ("DP", _I), ("VP", _I), ("k_offset", _I), ("v_offset", _I), ("i_offset", _I),
+                ("f_offset", _I), ("ld_row", _I), ("gate_cap", _F)]
+
+
+class Experts(ctypes.Structure):
+    """struct dh_experts: one layer's mixture of experts."""
+    _fields_ = [("hidden", _I), ("K", _I), ("experts", _I), ("top", _I), ("ff", _I), ("shared_ff", _I), ("eps", _F), ("limit", _F),
+                ("shared_limit", _F), ("d_norm", _P), ("d_layer_scale", _P), ("d_router", _P), ("d_up", _P), ("d_down", _P),
+                ("d_shared_up", _P), ("d_shared_down", _P)]
 
 
 def chain_phases(phases):
@@ -117,6 +137,8 @@ SIGNATURES = {
     "dh_attn_decode_qkv_kvlen_partials": (_I, [_P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _P, _I, _I, _I, _F, _I, _I, _F, _F,
                                                _I, _I, _I, _P]),
     "dh_dense_matmul": (_I, [_P, _I, _I, _P, _I, _I, _I, _I, _F, _P, _P, _P, _I, _I, _P, _I, _I, _I]),
+    "dh_dense_matmul_scaled": (_I, [_P, _I, _I, _P, _I, _I, _I, _I, _F, _P, _P, _P, _P, _I, _I, _P, _I, _I, _I]),
+    "dh_dense_gemv_scaled": (_I, [_P, _P, _I, _F, _P, _I, _I, _I, _F, _P, _P, _P, _P, _I, _P, _I]),
     "dh_dense_gemv": (_I, [_P, _P, _I, _F, _P, _I, _I, _I, _F, _P, _P, _P, _I, _P, _I]),
     "dh_dense_lmhead_argmax": (_I, [_P, _P, _I, _F, _P, _I, _I, _I, _F, _P, _P, _I, _P]),
     "dh_embed_sum": (_I, [_P, _I, _P, _P, _I, _P, _I64, _I64, _I64, _P, _I, _P, _I, _I, _I, _I, _P]),
@@ -124,6 +146,21 @@ SIGNATURES = {
     "dh_attn_spec_workspace_bytes": (_SZ, [_I, _I, _I]),
     "dh_attn_spec_kv_write": (_I, [ctypes.POINTER(AttnSpec), _P, _P, _P, _I, _I]),
     "dh_attn_spec_prefill": (_I, [ctypes.POINTER(AttnSpec), _P, _P, _P, _P, _I, _I, _I, _I]),
+    "dh_attn_spec_prefill_shared": (_I, [ctypes.POINTER(AttnSpec), _P, _P, _P, _I, _I, _P, _P, _I, _I, _I, _I]),
+    "dh_latent_rows": (_I, [ctypes.POINTER(Latent), _P, _P, _I, _I]),
+    "dh_latent_prefill_workspace_bytes": (_SZ, [ctypes.POINTER(Latent), _I, _I]),
+    "dh_latent_prefill": (_I, [ctypes.POINTER(Latent), _P, _P, _P, _P, _I, _I, _I, _I]),
+    "dh_latent_decode_workspace_bytes": (_SZ, [ctypes.POINTER(Latent), _I]),
+    "dh_latent_decode": (_I, [ctypes.POINTER(Latent), _P, _P, _P, _I, _P, _I, _P]),
+    "dh_mlstm_state_bytes": (_SZ, [ctypes.POINTER(MLSTM)]),
+    "dh_mlstm_step": (_I, [ctypes.POINTER(MLSTM), _P, _P, _P, _I, _P]),
+    "dh_mlstm_prefill_workspace_bytes": (_SZ, [ctypes.POINTER(MLSTM), _I]),
+    "dh_mlstm_prefill": (_I, [ctypes.POINTER(MLSTM), _P, _P, _P, _P, _I, _I, _I]),
+    "dh_head_norm_gate": (_I, [_P, _I, _P, _I, _P, _P, _I, _I, _I, _I, _I, _I, _F]),
+    "dh_experts_step_workspace_bytes": (_SZ, [ctypes.POINTER(Experts)]),
+    "dh_experts_step": (_I, [ctypes.POINTER(Experts), _P, _P]),
+    "dh_experts_prefill_workspace_bytes": (_SZ, [ctypes.POINTER(Experts), _I, _I]),
+    "dh_experts_prefill": (_I, [ctypes.POINTER(Experts), _P, _I, _P, _I, _P, _I]),
     "dh_attn_spec_decode": (_I, [ctypes.POINTER(AttnSpec), _P, _P, _P, _P, _I, _P, _I, _P]),
     "dh_rmsnorm": (_I, [_P, _P, _I, _P, _I, _I, _F, _I, _P, _P, _P, _F]),
     "dh_rmsnorm_sandwich_pair": (_I, [_P, _P, _P, _I, _P, _I, _P, _P, _I, _I, _F, _I]),

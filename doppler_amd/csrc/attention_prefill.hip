@@ -26,7 +26,8 @@
 // from stacked projection rows, every score loses r1 log2(1 + r2 (i - j)) (the distance bias in the softmax's own
 // units), value heads may differ in size from key heads (both are padded to the template's sizes with zeros in
 // LDS and registers), probabilities enter the second product as f16 high part + residual (22 bits), and the output is
-// gated per head and written in the operand type of the product that reads it.
+// gated per head and written in the operand type of the product that reads it.  A head's key may end in elements that all
+// heads of the token share (dh_attn_spec_prefill_shared): those come from rows of their own.
 // (Measured without effect at T = 2048..4096: a second LDS buffer per tile with one barrier per
 // tile instead of two, and dispatching the long late-query tiles first.)
 #include <algorithm>
@@ -70,6 +71,9 @@ struct PrefillArgs {
   float scale, softcap;
   // ---- SPEC form only
   int dk, dv;           // head sizes of caches and projection rows (<= the template's, multiples of 8)
+  int own_k;            // key elements of the head itself; the other dk - own_k are shared by all heads
+  const __half* KS;     // their rows, ld_shared apart
+  int64_t ld_shared;
   int64_t ld_q, ld_o;
   const float* r1;      // [H] or null
   const float* r2;
@@ -96,7 +100,8 @@ __global__ __launch_bounds__(256, SPEC ? 2 : 1) void attn_prefill_kernel(const P
   const int h = blockIdx.y, kvh = h / a.G;
   const int q0 = blockIdx.x * BQ;
   const int dk = SPEC ? a.dk : D, dv = SPEC ? a.dv : VD;
-  const int64_t k_stride = (int64_t)a.Hkv * dk, v_stride = (int64_t)a.Hkv * dv;
+  const int own_k = SPEC ? a.own_k : D;
+  const int64_t k_stride = (int64_t)a.Hkv * own_k, v_stride = (int64_t)a.Hkv * dv;
   int my_q[QT], my_pos[QT];                                   // query token of this lane's column, its absolute position
 #pragma unroll
   for (int u = 0; u < QT; u++) {
@@ -159,8 +164,11 @@ __global__ __launch_bounds__(256, SPEC ? 2 : 1) void attn_prefill_kernel(const P
     const int p_ = tid + 256 * r, key_ = p_ / (D / 8), c_ = p_ % (D / 8);                        \
     const int row_ = min(kbeg + (tile_) * BKEYS + key_, a.kv_len - 1);                           \
     kreg[r] = u32x4_t{0u, 0u, 0u, 0u};                                                           \
-    if (!SPEC || 8 * c_ < dk)                                                                    \
-      kreg[r] = *reinterpret_cast<const u32x4_t*>(a.K + (int64_t)row_ * k_stride + (int64_t)kvh * dk + 8 * c_); \
+    if (SPEC && 8 * c_ >= own_k) {                                                               \
+      if (8 * c_ < dk) kreg[r] = *reinterpret_cast<const u32x4_t*>(a.KS + (int64_t)row_ * a.ld_shared + 8 * c_ - own_k); \
+    } else {                                                                                     \
+      kreg[r] = *reinterpret_cast<const u32x4_t*>(a.K + (int64_t)row_ * k_stride + (int64_t)kvh * own_k + 8 * c_); \
+    }                                                                                            \
   }                                                                                              \
   _Pragma("unroll") for (int r = 0; r < VPIECES; r++) {                                          \
     const int vrow_ = min(kbeg + (tile_) * BKEYS + 2 * vpair + (r & 1), a.kv_len - 1);           \
@@ -368,9 +376,11 @@ namespace {
 template <int D, int VD>
 int launch_spec(const char* op, const PrefillArgs& a) {
   static const int env_qt = dh::tuning_int("DH_ATTN_SPEC_QT", 0);
-  const int qt = env_qt ? env_qt : dh::ceil_div(a.T, 128) * a.H >= 2 * dh::num_cus() ? 2 : 1;
+  // keys of more than 128 elements: two query groups would spill registers
+  const int qt = D > 128 ? 1 : env_qt ? env_qt : dh::ceil_div(a.T, 128) * a.H >= 2 * dh::num_cus() ? 2 : 1;
   const dim3 grid((unsigned)dh::ceil_div(a.T, 64 * qt), (unsigned)a.H);
-  if (qt == 2) hipLaunchKernelGGL((attn_prefill_kernel<D, VD, 2, true>), grid, dim3(256), 0, dh::stream(), a);
+  if constexpr (D > 128) hipLaunchKernelGGL((attn_prefill_kernel<D, VD, 1, true>), grid, dim3(256), 0, dh::stream(), a);
+  else if (qt == 2) hipLaunchKernelGGL((attn_prefill_kernel<D, VD, 2, true>), grid, dim3(256), 0, dh::stream(), a);
   else hipLaunchKernelGGL((attn_prefill_kernel<D, VD, 1, true>), grid, dim3(256), 0, dh::stream(), a);
   DH_CHECK_LAUNCH(op);
   return 0;
@@ -379,6 +389,12 @@ int launch_spec(const char* op, const PrefillArgs& a) {
 
 extern "C" int dh_attn_spec_prefill(const dh_attn_spec* spec, const float* d_qkv, const void* d_cache_k, const void* d_cache_v,
                                     void* d_out, int out_dtype, int ld_out, int T, int start_pos) {
+  return dh_attn_spec_prefill_shared(spec, d_qkv, d_cache_k, nullptr, 0, 0, d_cache_v, d_out, out_dtype, ld_out, T, start_pos);
+}
+
+extern "C" int dh_attn_spec_prefill_shared(const dh_attn_spec* spec, const float* d_qkv, const void* d_cache_k, const void* d_shared_k,
+                                           int shared_dim, int ld_shared, const void* d_cache_v, void* d_out, int out_dtype,
+                                           int ld_out, int T, int start_pos) {
   const char* op = "dh_attn_spec_prefill";
   DH_REQUIRE_INIT(op);
   if (int rc = dh::attn_spec_check(op, spec)) return rc;
@@ -389,17 +405,25 @@ extern "C" int dh_attn_spec_prefill(const dh_attn_spec* spec, const float* d_qkv
   if ((reinterpret_cast<uintptr_t>(d_qkv) | reinterpret_cast<uintptr_t>(d_cache_k) | reinterpret_cast<uintptr_t>(d_cache_v) |
        reinterpret_cast<uintptr_t>(d_out)) & 15)
     return dh::fail(1, "[%s] pointers must be 16-byte aligned", op);
-  if (spec->cache_dtype != DH_F16 || spec->D > 128 || spec->VD > 128)
-    return dh::attn_spec_prefill_general(op, spec, d_qkv, d_cache_k, d_cache_v, d_out, out_dtype, ld_out, T, start_pos);
+  const int dk = spec->D + shared_dim;
+  if (shared_dim < 0 || shared_dim % 8 || dk > 512) return dh::fail(1, "[%s] %d shared key elements beside %d must be a multiple of 8, 512 in all", op, shared_dim, spec->D);
+  if (shared_dim > 0 && (!d_shared_k || ld_shared < shared_dim || ld_shared % 8 || (reinterpret_cast<uintptr_t>(d_shared_k) & 15)))
+    return dh::fail(1, "[%s] shared key rows must be 16-byte aligned and ld_shared=%d a multiple of 8 that holds %d elements", op, ld_shared, shared_dim);
+  if (spec->ld_qkv < spec->H * dk) return dh::fail(1, "[%s] a projection row of %d floats does not hold its queries", op, spec->ld_qkv);
+  const dh::SharedKey shared{d_shared_k, shared_dim, ld_shared};
+  if (spec->cache_dtype != DH_F16 || dk > 256 || spec->VD > 128)
+    return dh::attn_spec_prefill_general(op, spec, d_qkv, d_cache_k, d_cache_v, d_out, out_dtype, ld_out, T, start_pos, shared);
   PrefillArgs a{};
   a.Q = d_qkv; a.K = static_cast<const __half*>(d_cache_k); a.V = static_cast<const __half*>(d_cache_v);
   a.O = out_dtype == DH_F32 ? static_cast<float*>(d_out) : nullptr;
   a.O16 = out_dtype == DH_BF16 ? static_cast<uint16_t*>(d_out) : nullptr;
   a.T = T; a.H = spec->H; a.Hkv = spec->Hkv; a.G = spec->H / spec->Hkv; a.kv_len = start_pos + T; a.start_pos = start_pos;
   a.causal = 1; a.window = spec->window; a.scale = spec->scale; a.softcap = 0.f;
-  a.dk = spec->D; a.dv = spec->VD; a.ld_q = spec->ld_qkv; a.ld_o = ld_out;
+  a.dk = dk; a.dv = spec->VD; a.own_k = spec->D; a.KS = static_cast<const __half*>(d_shared_k); a.ld_shared = ld_shared;
+  a.ld_q = spec->ld_qkv; a.ld_o = ld_out;
   a.r1 = spec->d_bias_r1; a.r2 = spec->d_bias_r2;
   a.gate = spec->gate_offset >= 0 ? d_qkv + spec->gate_offset : nullptr;
-  if (spec->D <= 64) return spec->VD <= 64 ? launch_spec<64, 64>(op, a) : launch_spec<64, 128>(op, a);
-  return spec->VD <= 64 ? launch_spec<128, 64>(op, a) : launch_spec<128, 128>(op, a);
+  if (dk <= 64) return spec->VD <= 64 ? launch_spec<64, 64>(op, a) : launch_spec<64, 128>(op, a);
+  if (dk <= 128) return spec->VD <= 64 ? launch_spec<128, 64>(op, a) : launch_spec<128, 128>(op, a);
+  return dk <= 192 ? launch_spec<192, 128>(op, a) : launch_spec<256, 128>(op, a);
 }

@@ -33,7 +33,10 @@ struct SpecArgs {
   uint16_t* O16;        // bf16 output rows
   float* ws;            // [H][nsplit of the launch][VD + 2]
   int64_t ld_qkv, ld_out;
-  int H, Hkv, G, D, VD, value_dim;
+  int H, Hkv, G, D, VD, value_dim;      // D: key elements of a head, its own and the shared ones
+  int own_d;                            // its own
+  const void* KS;                       // rows of the shared ones, ld_shared apart
+  int64_t ld_shared;
   int k_off, v_off, gate_off;
   int pos0;             // position of the first query token
   int window, kbeg, kend, nsplit;
@@ -128,9 +131,10 @@ __global__ __launch_bounds__(256) void attn_spec_kernel(const SpecArgs a_in) {
     kbeg = a.window > 0 ? max(0, pos - a.window + 1) : 0;
   }
   const float* row = a.qkv + (int64_t)t * a.ld_qkv;
-  const KV* Kc = static_cast<const KV*>(a.K) + (int64_t)kvh * a.D + 8 * piece;
+  const bool own = 8 * piece < a.own_d;
+  const KV* Kc = own ? static_cast<const KV*>(a.K) + (int64_t)kvh * a.own_d + 8 * piece : static_cast<const KV*>(a.KS) + 8 * piece - a.own_d;
   const KV* Vc = static_cast<const KV*>(a.V) + (int64_t)kvh * a.VD + 8 * piece;
-  const int64_t kstride = (int64_t)a.Hkv * a.D, vstride = (int64_t)a.Hkv * a.VD;
+  const int64_t kstride = own ? (int64_t)a.Hkv * a.own_d : a.ld_shared, vstride = (int64_t)a.Hkv * a.VD;
   const bool has_k = 8 * piece < a.D, has_v = 8 * piece < a.VD;
   const int nchunks = (kend - kbeg + CH - 1) / CH;
 
@@ -371,13 +375,13 @@ SpecKernel pick_lanes(int lanes, int gt) {
   }
 }
 
-int lanes_for(const dh_attn_spec* s) {
-  const int n = std::max(s->D, s->VD);
+int lanes_for(int D, int VD) {
+  const int n = std::max(D, VD);
   return n <= 64 ? 8 : n <= 128 ? 16 : n <= 256 ? 32 : 64;
 }
-int heads_at_once(const dh_attn_spec* s) {
-  const int G = s->H / s->Hkv, gt = G <= 1 ? 1 : G <= 2 ? 2 : G <= 4 ? 4 : 8;
-  return lanes_for(s) == 64 ? std::min(gt, 4) : gt;      // wide heads: fewer of them at once fit the registers
+int heads_at_once(int G, int lanes) {
+  const int gt = G <= 1 ? 1 : G <= 2 ? 2 : G <= 4 ? 4 : 8;
+  return lanes == 64 ? std::min(gt, 4) : gt;      // wide heads: fewer of them at once fit the registers
 }
 
 SpecArgs make_args(const dh_attn_spec* s, const float* qkv, void* K, void* V) {
@@ -386,13 +390,14 @@ SpecArgs make_args(const dh_attn_spec* s, const float* qkv, void* K, void* V) {
   a.ld_qkv = s->ld_qkv;
   a.H = s->H; a.Hkv = s->Hkv; a.G = s->H / s->Hkv; a.D = s->D; a.VD = s->VD; a.value_dim = s->value_dim;
   a.k_off = s->k_offset; a.v_off = s->v_offset; a.gate_off = s->gate_offset;
+  a.own_d = s->D;
   a.window = s->window; a.value_norm = s->value_norm; a.scale = s->scale; a.value_eps = s->value_eps;
   a.r1 = s->d_bias_r1; a.r2 = s->d_bias_r2;
   return a;
 }
 
 int launch_spec(const char* op, const dh_attn_spec* s, const SpecArgs& a, int T) {
-  const int gt = heads_at_once(s), lanes = lanes_for(s);
+  const int lanes = lanes_for(a.D, a.VD), gt = heads_at_once(a.G, lanes);
   const dim3 grid((unsigned)(s->Hkv * dh::ceil_div(a.G, gt)), (unsigned)a.nsplit, (unsigned)T);
   SpecKernel k = s->cache_dtype == DH_F16 ? pick_lanes<__half>(lanes, gt) : pick_lanes<float>(lanes, gt);
   hipLaunchKernelGGL(k, grid, dim3(256), 0, dh::stream(), a);
@@ -421,11 +426,12 @@ int attn_spec_check(const char* op, const dh_attn_spec* s) {
 }
 
 int attn_spec_prefill_general(const char* op, const dh_attn_spec* s, const float* d_qkv, const void* K, const void* V,
-                              void* d_out, int out_dtype, int ld_out, int T, int start_pos) {
+                              void* d_out, int out_dtype, int ld_out, int T, int start_pos, const SharedKey& shared) {
   SpecArgs a = make_args(s, d_qkv, const_cast<void*>(K), const_cast<void*>(V));
   a.O = out_dtype == DH_F32 ? static_cast<float*>(d_out) : nullptr;
   a.O16 = out_dtype == DH_BF16 ? static_cast<uint16_t*>(d_out) : nullptr;
   a.ld_out = ld_out; a.nsplit = 1; a.direct = 1;
+  a.D += shared.dim; a.KS = shared.rows; a.ld_shared = shared.ld;
   // the grid's third dimension holds at most 65535 query tokens
   for (int t0 = 0; t0 < T; t0 += 32768) {
     SpecArgs b = a;

@@ -26,6 +26,7 @@ __device__ __forceinline__ float activate(float z, int act) {
   }
   if (act == DH_ACT_SILU) return z / (1.0f + __expf(-z));
   if (act == DH_ACT_GELU) return 0.5f * z * (1.0f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z)));
+  if (act == DH_ACT_GELU_ERF) return 0.5f * z * (1.0f + erff(0.7071067811865476f * z));
   return z;
 }
 

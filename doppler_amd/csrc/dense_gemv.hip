@@ -6,7 +6,7 @@
 // before the row is prepared and travels meanwhile.  The row is kept as two planes of 16-byte pieces (elements
 // 0..3 and 4..7 of every eight) so that a wave's reads of either plane are consecutive.
 //
-// Outputs as in the multi-row product (dense_gemm.hip): columns below n_first with bias and residual, the rest
+// Outputs as in the multi-row product (dense_gemm.hip): columns below n_first with bias, column scale and residual, the rest
 // through an activation; or the argmax over all of them (output head).
 #include <algorithm>
 #include <cfloat>
@@ -31,6 +31,7 @@ struct GemvArgs {
   float alpha;
   const float* bias;
   const float* residual;
+  const float* col_scale;
   float* C;
   int n_first;
   float* C2;
@@ -129,6 +130,7 @@ __global__ __launch_bounds__(64 * WAVES) void gemv_kernel(const GemvArgs a) {
         if (lane == 0 && n < a.N) {
           if (n < a.n_first) {
             float y = v + (a.bias ? a.bias[n] : 0.f);
+            if (a.col_scale) y *= a.col_scale[n];
             if (a.residual) y += a.residual[n];
             if (a.C) a.C[n] = y;
           } else {
@@ -217,6 +219,13 @@ extern "C" {
 int dh_dense_gemv(const float* d_x, const float* d_norm_weight, int hidden, float eps, const void* d_W, int ldw, int N,
                   int K, float alpha, const float* d_bias, const float* d_residual, float* d_C, int n_first, float* d_C2,
                   int activation) {
+  return dh_dense_gemv_scaled(d_x, d_norm_weight, hidden, eps, d_W, ldw, N, K, alpha, d_bias, nullptr, d_residual, d_C, n_first, d_C2,
+                              activation);
+}
+
+int dh_dense_gemv_scaled(const float* d_x, const float* d_norm_weight, int hidden, float eps, const void* d_W, int ldw, int N,
+                         int K, float alpha, const float* d_bias, const float* d_col_scale, const float* d_residual, float* d_C,
+                         int n_first, float* d_C2, int activation) {
   const char* op = "dh_dense_gemv";
   DH_REQUIRE_INIT(op);
   if (int rc = check(op, d_x, d_norm_weight, hidden, eps, d_W, ldw, N, K)) return rc;
@@ -224,7 +233,7 @@ int dh_dense_gemv(const float* d_x, const float* d_norm_weight, int hidden, floa
   if ((n_first > 0 && !d_C) || (n_first < N && !d_C2)) return dh::fail(1, "[%s] null output pointer", op);
   if (d_x == d_C || d_x == d_C2) return dh::fail(1, "[%s] an output must not be the activation row", op);
   GemvArgs a = make_args(d_x, d_norm_weight, hidden, eps, d_W, ldw, N, K, alpha);
-  a.bias = d_bias; a.residual = d_residual; a.C = d_C; a.n_first = n_first; a.C2 = d_C2; a.act = activation;
+  a.bias = d_bias; a.col_scale = d_col_scale; a.residual = d_residual; a.C = d_C; a.n_first = n_first; a.C2 = d_C2; a.act = activation;
   return dispatch<false>(op, a, nullptr);
 }
 

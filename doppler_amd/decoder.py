@@ -53,7 +53,10 @@ class DecoderBase:
     and device_kv_len_served (whether captured steps can read the key count on the device).
 
     The state of the sequence besides its cache rows is the tokens themselves (`history`): a model whose embedding
-    reads the previous token finds it there at every portion's start.  A sequence starts when position 0 is fed."""
+    reads the previous token finds it there at every portion's start.  A sequence starts when position 0 is fed.
+
+    A model whose layers carry recurrent state returns its buffers from _recurrent_state().  That state stands behind the last
+    token fed and cannot be taken back: positions must follow one another, and one that does not is refused."""
     TOKEN_RING = 64      # tokens one decode_batch submit can produce
     device_kv_len_served = True
     UNSERVED_CAPTURE = "capture_step serves the step with the key count on the device"
@@ -78,6 +81,17 @@ class DecoderBase:
         self._input_ptr = self.ids.data_ptr()
         self.history = np.zeros(max_seq, np.uint32)
         self.length = 0      # tokens of the sequence fed through feed()
+        self._state_pos = 0  # the position recurrent state is ready for
+        self._capturing = False
+
+    def _recurrent_state(self):
+        return []
+
+    def _advance(self, pos, tokens):
+        """Recurrent state moves from position pos over so many tokens."""
+        if pos not in (0, self._state_pos) and self._recurrent_state():
+            raise ValueError("the sequence's recurrent state stands at position %d, not at %d" % (self._state_pos, pos))
+        self._state_pos = pos + tokens
 
     def _remember(self, pos, tokens):
         tokens = np.atleast_1d(np.asarray(tokens, np.uint32))[:max(0, self.max_seq - pos)]
@@ -98,6 +112,8 @@ class DecoderBase:
             # the ops take no cache capacity: a position past the caches would write K/V and read
             # the position tables out of bounds
             raise ValueError("decode position %d is outside the KV cache (max_seq=%d)" % (pos, self.max_seq))
+        if not self._capturing:
+            self._advance(pos, 1)
         if from_device_token:
             ids_ptr, prev_ptr = self.token.data_ptr() + 4 * in_index, self._input_ptr
         else:
@@ -221,8 +237,16 @@ class DecoderBase:
         # with the guard on the captured step also clears the status words and leaves its token next
         # to them (the library moves the checks' step number with the position at every replay)
         out_index = self.TOKEN_RING - 1 if self.finiteness_guard else 0
+        state = self._recurrent_state()
+        before, kept = self._state_pos, [t.clone() for t in state]
+        torch.cuda.synchronize()
+        self._state_pos = pos
         self.enqueue_step(pos, want_logits, out_index=out_index)
         capi.check(self.L.dh_sync())
+        for t, k in zip(state, kept):        # that run belongs to no sequence
+            t.copy_(k)
+        torch.cuda.synchronize()
+        self._state_pos = before
         self._graph_device_kv_len = bool(device_kv_len)
         capi.check(self.L.dh_graph_begin())
         g = ctypes.c_void_p()
@@ -250,6 +274,7 @@ class DecoderBase:
             raise ValueError("decode position %d is outside the KV cache (max_seq=%d)" % (pos, self.max_seq))
         if getattr(self, "_graph", None) is None:
             self.capture_step(pos)
+        self._advance(pos, 1)
         self.set_token(token, pos + 1, pos=pos)
         capi.check(self.L.dh_graph_launch(self._graph, pos))
         if pos + 1 < self.max_seq and not self._graph_device_kv_len:
@@ -310,6 +335,7 @@ class DecoderBase:
         out = [None] * len(want) if want is not None else None
         for c0 in range(0, tokens.size, chunk):
             ids = np.ascontiguousarray(tokens[c0:c0 + chunk])
+            self._advance(start_pos + c0, ids.size)
             base, stride = self._prefill_chunk(ids, start_pos + c0, chunk)
             if want is not None:
                 at = [i for i, w in enumerate(want) if c0 <= w < c0 + ids.size]

@@ -1,6 +1,7 @@
-"""Decoder with dense bf16 weights: parallel layers of attention and feed-forward, described layer by layer.
+"""Decoder with dense bf16 weights, described layer by layer.  Layers are parallel (attention and feed-forward side by side, below) or
+sequential (sublayers one after the other: sublayers.py); embedding, head, portions and state are the same for both.
 
-A layer is  x <- x + mixer(norm(x)) + ff(norm(x)).  Both sublayers read one normed row, and both results are added to
+A parallel layer is  x <- x + mixer(norm(x)) + ff(norm(x)).  Both sublayers read one normed row, and both results are added to
 the residual, so a layer is two products:
 
     [ q | k | v | gate | up ] = W_in norm(x)         one stacked product; `up` leaves it through the activation
@@ -24,18 +25,7 @@ import torch
 
 from . import capi
 from .decoder import DecoderBase, _dev_bytes
-
-ACTIVATIONS = {"relu2": capi.ACT_RELU2, "silu": capi.ACT_SILU, "gelu_tanh": capi.ACT_GELU, None: capi.ACT_NONE}
-GEMV_MAX_K = 32768
-
-
-def _up(n, m):
-    return (n + m - 1) // m * m
-
-
-def bf16_to_f32(bits):
-    return (np.ascontiguousarray(bits, np.uint16).astype(np.uint32) << 16).view(np.float32)
-
+from .sublayers import ACTIVATIONS, GEMV_MAX_K, Scratch, SequentialLayer, _up, bf16_to_f32, rotary_tables
 
 def f32_to_bf16(x):
     """Round to nearest even; returns uint16 bit patterns."""
@@ -84,9 +74,11 @@ class DenseDecoder(DecoderBase):
         """cfg: dict(hidden, vocab, eps, logit_scale, max_positions (0: no position table),
         bigram=dict(buckets, mul_prev, mul_cur) or None,
         layers=[dict(mixer=dict(heads, kv_heads, dim, vdim, window (0: none), scale, log_bias, value_norm, gate),
-                     mlp=dict(ff, activation) or None)]);
+                     mlp=dict(ff, activation) or None), or a sequential layer: dict(sequential=True, mixer=dict(type, ..),
+                     mlp=dict(type, ..) or None)]);
         weights: dict(embed, bigram, pos, head: bf16 bits [rows, hidden]; final_norm f32;
-        layers=[dict(norm, q_bias, k_bias, v_bias, bias_r1, bias_r2: f32; q, k, v, gate, o, up, down: bf16 bits [out, in])])."""
+        layers=[dict(norm, q_bias, k_bias, v_bias, bias_r1, bias_r2: f32; q, k, v, gate, o, up, down: bf16 bits [out, in]), or for a
+        sequential layer what SequentialLayer takes])."""
         if compute not in ("bf16", "f32"):
             raise ValueError("compute must be 'bf16' or 'f32', got %r" % (compute,))
         if cfg["max_positions"] and max_seq > cfg["max_positions"]:
@@ -106,9 +98,15 @@ class DenseDecoder(DecoderBase):
             out[:Hd] = v
             return _dev_bytes(out)
 
+        self.x = f32(self.kx)                 # residual stream of the step
+        self.scratch = Scratch()
+        self._rotary = {}
         self.layers = []
         ws = 256
         for spec, w in zip(self.cfg["layers"], weights["layers"]):
+            if spec.get("sequential"):
+                self.layers.append(SequentialLayer(self, spec, w, self.layers))
+                continue
             m, mlp = spec["mixer"], spec["mlp"]
             w_in, bias, w_out, g = stack_layer(m, mlp, w, Hd)
             d = dict(geo=g, w_in=_dev_bytes(w_in), bias=_dev_bytes(bias), w_out=_dev_bytes(w_out), norm=padded_f32(w["norm"]),
@@ -133,16 +131,28 @@ class DenseDecoder(DecoderBase):
         head[:, :Hd] = weights["head"]
         self.head = _dev_bytes(head)
         self.final_norm = padded_f32(weights["final_norm"])
-        self.qkv_n = max([d["geo"]["n_first"] for d in self.layers] + [1])
-        self.x = f32(self.kx)                 # residual stream of the step
+        self.recurrent = [t for d in self.layers if isinstance(d, SequentialLayer) for t in d.state()]
+        self.qkv_n = max([d["geo"]["n_first"] for d in self._parallel()] + [1])
         self.qkv = f32(self.qkv_n)
         # [attention | act] rows: one buffer per layer shape, so that the padding behind the columns stays zero
         self.mixed = {s: f32(s[1]) for s in self._mixed_shapes()}
         self._pf_rows = 0
         torch.cuda.synchronize()
 
+    def _parallel(self):
+        return [d for d in self.layers if not isinstance(d, SequentialLayer)]
+
+    def _recurrent_state(self):
+        return self.recurrent
+
+    def rotary(self, base, dims):
+        """Device tables of the rotary angles of every position the cache holds, shared by layers with equal rotations."""
+        if (base, dims) not in self._rotary:
+            self._rotary[base, dims] = tuple(_dev_bytes(t) for t in rotary_tables(base, dims, self.max_seq))
+        return self._rotary[base, dims]
+
     def _mixed_shapes(self):
-        return {self._mixed_key(d["geo"]) for d in self.layers}
+        return {self._mixed_key(d["geo"]) for d in self._parallel()}
 
     @staticmethod
     def _mixed_key(geo):
@@ -153,6 +163,9 @@ class DenseDecoder(DecoderBase):
         elem = 2 if self.compute == "bf16" else 4
         total = self.cfg["vocab"] * self.cfg["hidden"] * 2
         for spec, d in zip(self.cfg["layers"], self.layers):
+            if isinstance(d, SequentialLayer):
+                total += d.step_bytes(ctx)
+                continue
             m, g = spec["mixer"], d["geo"]
             rows = min(ctx, m["window"]) if m["window"] else ctx
             total += 2 * self.cfg["hidden"] * (g["n"] + g["attn_cols"] + g["ff"]) + rows * m["kv_heads"] * (g["D"] + g["VD"]) * elem
@@ -177,26 +190,31 @@ class DenseDecoder(DecoderBase):
         L, c, ck = self.L, self.cfg, capi.check
         kv_len = self.ids.data_ptr() + 4 if device_kv_len else None
         for li, d in enumerate(self.layers):
-            g = d["geo"]
-            mixed = self.mixed[self._mixed_key(g)]
-            act = mixed.data_ptr() + 4 * g["attn_cols"] if g["ff"] else None
-            if g["kx"] <= GEMV_MAX_K:
-                ck(L.dh_dense_gemv(self.x.data_ptr(), d["norm"].data_ptr(), c["hidden"], c["eps"], d["w_in"].data_ptr(), g["kx"],
-                                   g["n"], g["kx"], 1.0, d["bias"].data_ptr(), None, self.qkv.data_ptr(), g["n_first"], act,
-                                   d["act"]))
+            if isinstance(d, SequentialLayer):
+                d.step(pos, kv_len)
             else:
-                self._enqueue_in(d, self.x.data_ptr(), self._wide_row().data_ptr(), capi.F32, self.qkv.data_ptr(), act, 1, g["k2"])
-            ck(L.dh_attn_spec_decode(ctypes.byref(d["spec"]), self.qkv.data_ptr(), d["cache_k"].data_ptr(),
-                                     d["cache_v"].data_ptr(), mixed.data_ptr(), pos, kv_len, self.max_seq,
-                                     self.attn_ws.data_ptr()))
-            if g["k2"] <= GEMV_MAX_K:
-                ck(L.dh_dense_gemv(mixed.data_ptr(), None, 0, 0.0, d["w_out"].data_ptr(), g["k2"], c["hidden"], g["k2"], 1.0,
-                                   None, self.x.data_ptr(), self.x.data_ptr(), c["hidden"], None, capi.ACT_NONE))
-            else:
-                self._enqueue_out(d, mixed.data_ptr(), capi.F32, self.x.data_ptr(), 1)
+                self._step_parallel(d, pos, kv_len)
             if self.finiteness_guard:
                 ck(L.dh_check_finiteness(self.x.data_ptr(), capi.F32, c["hidden"], self.token.data_ptr() + 4 * self.TOKEN_RING,
                                          li, pos, self.finiteness_abs_threshold))
+
+    def _step_parallel(self, d, pos, kv_len):
+        L, c, ck, g = self.L, self.cfg, capi.check, d["geo"]
+        mixed = self.mixed[self._mixed_key(g)]
+        act = mixed.data_ptr() + 4 * g["attn_cols"] if g["ff"] else None
+        if g["kx"] <= GEMV_MAX_K:
+            ck(L.dh_dense_gemv(self.x.data_ptr(), d["norm"].data_ptr(), c["hidden"], c["eps"], d["w_in"].data_ptr(), g["kx"],
+                               g["n"], g["kx"], 1.0, d["bias"].data_ptr(), None, self.qkv.data_ptr(), g["n_first"], act, d["act"]))
+        else:
+            self._enqueue_in(d, self.x.data_ptr(), self._wide_row().data_ptr(), capi.F32, self.qkv.data_ptr(), act, 1, g["k2"])
+        ck(L.dh_attn_spec_decode(ctypes.byref(d["spec"]), self.qkv.data_ptr(), d["cache_k"].data_ptr(),
+                                 d["cache_v"].data_ptr(), mixed.data_ptr(), pos, kv_len, self.max_seq,
+                                 self.attn_ws.data_ptr()))
+        if g["k2"] <= GEMV_MAX_K:
+            ck(L.dh_dense_gemv(mixed.data_ptr(), None, 0, 0.0, d["w_out"].data_ptr(), g["k2"], c["hidden"], g["k2"], 1.0,
+                               None, self.x.data_ptr(), self.x.data_ptr(), c["hidden"], None, capi.ACT_NONE))
+        else:
+            self._enqueue_out(d, mixed.data_ptr(), capi.F32, self.x.data_ptr(), 1)
 
     def _wide_row(self):
         if getattr(self, "_wide", None) is None:
@@ -250,6 +268,9 @@ class DenseDecoder(DecoderBase):
         ck(L.dh_embed_sum(b["ids"].data_ptr(), 1, b["ids"].data_ptr(), *self._embed_args(), x, self.kx, T, c["hidden"], pos, None))
         elem = b["normed"].element_size()
         for d in self.layers:
+            if isinstance(d, SequentialLayer):
+                d.rows(x, T, pos)
+                continue
             g = d["geo"]
             mixed = b["mixed"][self._mixed_key(g)].data_ptr()
             self._enqueue_in(d, x, b["normed"].data_ptr(), self.operand, b["qkv"].data_ptr(),

@@ -39,9 +39,15 @@ def _load_zepavik(directory, max_seq, dtype, **kwargs):
     return zepavik.load_decoder(directory, max_seq, dtype, **kwargs)
 
 
+def _load_gusolorn(directory, max_seq, dtype, **kwargs):
+    from . import gusolorn
+    return gusolorn.load_decoder(directory, max_seq, dtype, **kwargs)
+
+
 RDRR = Model("RDRR Q4_K", ["bfloat16"], _load_rdrr)
 ARCHITECTURES = {
     "Zepavik": Model("Zepavik", ["bfloat16", "float32"], _load_zepavik, library="dense"),
+    "Gusolorn": Model("Gusolorn", ["bfloat16", "float32"], _load_gusolorn, library="dense"),
 }
 
 

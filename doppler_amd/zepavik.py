@@ -8,33 +8,11 @@ closed with its name.
 import json
 import os
 
+from .config_fields import ConfigError, count as _count, take as _take
 from .dense_decoder import DenseDecoder, bf16_to_f32, f32_to_bf16
 from .safetensors_file import SafetensorsFile, write_safetensors
 
 ARCHITECTURE = "Zepavik"
-
-
-class ConfigError(ValueError):
-    pass
-
-
-def _take(obj, where, required, optional=()):
-    if not isinstance(obj, dict):
-        raise ConfigError("%s must be an object, got %r" % (where, obj))
-    unknown = sorted(set(obj) - set(required) - set(optional))
-    if unknown:
-        raise ConfigError("%s has keys this design does not have: %s" % (where, ", ".join(unknown)))
-    missing = sorted(set(required) - set(obj))
-    if missing:
-        raise ConfigError("%s lacks %s" % (where, ", ".join(missing)))
-    return obj
-
-
-def _count(obj, key, where, low=1):
-    v = obj[key]
-    if isinstance(v, bool) or not isinstance(v, int) or v < low:
-        raise ConfigError("%s.%s must be an integer of at least %d, got %r" % (where, key, low, v))
-    return v
 
 
 def decoder_config(config):

@@ -40,6 +40,7 @@ extern "C" {
 #define DH_ACT_SILU 0
 #define DH_ACT_GELU 1
 #define DH_ACT_RELU2 2   /* max(z, 0)^2: plain activations of the dense products only */
+#define DH_ACT_GELU_ERF 3   /* the exact gelu, 0.5 z (1 + erf(z / sqrt 2)): the same */
 #define DH_ACT_NONE (-1)
 
 #define DH_KV_CONTIGUOUS 0
@@ -367,6 +368,11 @@ int dh_attn_decode_qkv_kvlen_partials(const float* d_qkv, const float* d_q_weigh
 int dh_dense_matmul(const void* d_A, int a_dtype, int lda, const void* d_W, int ldw, int M, int N, int K, float alpha,
                     const float* d_bias, const float* d_residual, float* d_C, int ldc, int n_first, void* d_C2,
                     int c2_dtype, int ldc2, int activation);
+/* The same with C[m][n] = (alpha * acc + bias[n]) * col_scale[n] + residual[m][n].  In both forms f16 activations (a_dtype
+ * DH_F16) stand for f16 weights as well, and c2_dtype may be DH_F16. */
+int dh_dense_matmul_scaled(const void* d_A, int a_dtype, int lda, const void* d_W, int ldw, int M, int N, int K, float alpha,
+                           const float* d_bias, const float* d_col_scale, const float* d_residual, float* d_C, int ldc,
+                           int n_first, void* d_C2, int c2_dtype, int ldc2, int activation);
 
 /* The same product for ONE f32 activation row (decode; HBM-bound), d_C2 in f32, with an optional RMSNorm of the
  * row in its prologue: x * rsqrt(mean of the first `hidden` elements squared + eps) * w.  d_x and d_norm_weight
@@ -374,6 +380,9 @@ int dh_dense_matmul(const void* d_A, int a_dtype, int lda, const void* d_W, int 
 int dh_dense_gemv(const float* d_x, const float* d_norm_weight, int hidden, float eps, const void* d_W, int ldw, int N,
                   int K, float alpha, const float* d_bias, const float* d_residual, float* d_C, int n_first, float* d_C2,
                   int activation);
+int dh_dense_gemv_scaled(const float* d_x, const float* d_norm_weight, int hidden, float eps, const void* d_W, int ldw, int N,
+                         int K, float alpha, const float* d_bias, const float* d_col_scale, const float* d_residual, float* d_C,
+                         int n_first, float* d_C2, int activation);
 /* dh_lmhead_argmax_f16_rmsnorm for an untied bf16 head: logits = alpha * W norm(x), token = their argmax (ties to
  * the lowest index).  d_workspace: dh_lmhead_argmax_workspace_bytes(vocab). */
 int dh_dense_lmhead_argmax(const float* d_x, const float* d_norm_weight, int hidden, float eps, const void* d_W, int ldw,
@@ -428,6 +437,94 @@ int dh_attn_spec_prefill(const dh_attn_spec* spec, const float* d_qkv, const voi
 size_t dh_attn_spec_workspace_bytes(int H, int VD, int max_kv_len);
 int dh_attn_spec_decode(const dh_attn_spec* spec, const float* d_qkv, void* d_cache_k, void* d_cache_v, float* d_out,
                         int pos, const uint32_t* d_kv_len, int max_kv_len, void* d_workspace);
+/* dh_attn_spec_prefill for keys that end in elements all heads share: head h's key at row r is [cache_k[r][h] (D elements) |
+ * shared_k + r * ld_shared (shared_dim elements)], its query D + shared_dim floats at h * (D + shared_dim). */
+int dh_attn_spec_prefill_shared(const dh_attn_spec* spec, const float* d_qkv, const void* d_cache_k, const void* d_shared_k,
+                                int shared_dim, int ld_shared, const void* d_cache_v, void* d_out, int out_dtype, int ld_out,
+                                int T, int start_pos);
+
+/* ---- attention over a low-rank latent ----
+ *   k_h = [W_uk,h c | k_rot],  v_h = W_uv,h c,  softmax over 0 <= i - j < window of scale * (q_h . k_h)
+ * A cache row is [c (C elements) | k_rot (R elements)], f16 or f32, one per position, for all heads; c is the raw latent divided by
+ * its root mean square and weighted, k_rot and the end of every query are turned by interleaved rotary positions
+ * (tables cos/sin [position][rot_dim / 2]).
+ * Padded sizes (zeros behind the real elements): D and VD multiples of 8, R of 32, C of 64, D + R and VD at most 512.  A projection
+ * row holds H queries of D + R floats and, at dkv_offset, the raw [c | k_rot] in C + R floats; dkv_offset < 0: another layer writes
+ * the cache rows.
+ * Up projections: d_uk [H * D][C] and d_uv [H * VD][C] in the cache's operand type (f16, or bf16 beside f32 caches) for portions,
+ * d_uk_t [H][C][D] and d_uv_rows [H * VD][C] in bf16 for single tokens. */
+typedef struct dh_latent {
+  int H, D, R, VD, rank, C, rot_dim;
+  int window;
+  int cache_dtype;
+  int dkv_offset, ld_row;
+  float scale, eps;
+  const float* d_latent_norm;   /* [rank] */
+  const float* d_cos;
+  const float* d_sin;
+  const void* d_uk;
+  const void* d_uv;
+  const void* d_uk_t;
+  const void* d_uv_rows;
+} dh_latent;
+/* A portion's rows: queries rotated in place, cache rows start_pos .. written (unless another layer writes them). */
+int dh_latent_rows(const dh_latent* spec, float* d_rows, void* d_cache, int T, int start_pos);
+/* T queries (rotated rows) at positions start_pos .. against the cache rows up to their own.  Output as dh_attn_spec_prefill. */
+size_t dh_latent_prefill_workspace_bytes(const dh_latent* spec, int T, int start_pos);
+int dh_latent_prefill(const dh_latent* spec, const float* d_rows, const void* d_cache, void* d_workspace, void* d_out, int out_dtype,
+                      int ld_out, int T, int start_pos);
+/* One step from its raw projection row: the cache row is appended, d_out is [H * VD] f32.  d_kv_len as in dh_attn_spec_decode. */
+size_t dh_latent_decode_workspace_bytes(const dh_latent* spec, int max_kv_len);
+int dh_latent_decode(const dh_latent* spec, const float* d_row, void* d_cache, float* d_out, int pos, const uint32_t* d_kv_len,
+                     int max_kv_len, void* d_workspace);
+
+/* ---- matrix memory with exponential gates (mLSTM) ----
+ *   i = cap tanh(z_i / cap), f = log sigmoid(cap tanh(z_f / cap)), m' = max(f + m, i)
+ *   S' = e^(f + m - m') S + e^(i - m') k v^T,  n' likewise with k,  o = S'^T q / (max(|n' . q|, e^-m') + 1e-6)
+ * q is divided by sqrt(dim) here.  Everything is 32-bit.  Projection rows of ld_row floats: H queries of DP floats at 0, keys at
+ * k_offset, H values of VP floats at v_offset, the gates' H numbers at i_offset and f_offset; DP and VP are dim and vdim padded to
+ * multiples of 32 with zeros.  The state (dh_mlstm_state_bytes) counts as zero at position 0. */
+typedef struct dh_mlstm {
+  int H, dim, vdim, DP, VP;
+  int k_offset, v_offset, i_offset, f_offset, ld_row;
+  float gate_cap;
+} dh_mlstm;
+size_t dh_mlstm_state_bytes(const dh_mlstm* spec);
+/* One step: d_out is [H * VP].  d_kv_len (may be NULL): the position is *d_kv_len - 1. */
+int dh_mlstm_step(const dh_mlstm* spec, const float* d_row, void* d_state, float* d_out, int pos, const uint32_t* d_kv_len);
+/* T tokens at positions start_pos ..: outputs [T][ld_out], the state moves behind the last one. */
+size_t dh_mlstm_prefill_workspace_bytes(const dh_mlstm* spec, int T);
+int dh_mlstm_prefill(const dh_mlstm* spec, const float* d_rows, void* d_state, void* d_workspace, float* d_out, int ld_out, int T,
+                     int start_pos);
+/* y = x_h / sqrt(mean of the head's `size` elements squared + eps) * weight * sigmoid(gate), per head of `padded` elements;
+ * output DH_BF16 or DH_F32. */
+int dh_head_norm_gate(const float* d_x, int ld_x, const float* d_gate, int ld_gate, const float* d_weight, void* d_out, int out_dtype,
+                      int ld_out, int rows, int H, int padded, int size, float eps);
+
+/* ---- mixture of experts with clamped gates ----
+ *   h = norm(x), z = W_router h, s = sigmoid(z); the `top` largest are chosen (ties: the lower index)
+ *   x += ls * (sum over chosen e of expert_e(s_e h) + sigmoid(z_E) expert_shared(h))
+ *   expert(y) = W_down (g sigmoid(1.702 g) (clamp(u, +-limit) + 1)),  g = min(W_gate y, limit), u = W_up y
+ * Matrices are bf16: d_router [experts (+ 1 for the shared expert's number)][K]; d_up [experts][2 ff][K] with 32 gate rows, 32 up rows,
+ * 32 gate rows, ..; d_down [experts][hidden][ff]; the shared ones alike with shared_ff (0: no shared expert).  ff and shared_ff are
+ * padded to multiples of 64, K holds hidden padded to a multiple of 64; d_norm has K floats. */
+typedef struct dh_experts {
+  int hidden, K, experts, top, ff, shared_ff;
+  float eps, limit, shared_limit;
+  const float* d_norm;
+  const float* d_layer_scale;   /* [hidden], NULL: ones */
+  const void* d_router;
+  const void* d_up;
+  const void* d_down;
+  const void* d_shared_up;
+  const void* d_shared_down;
+} dh_experts;
+/* One residual row d_x [K] (zeros behind hidden), updated in place. */
+size_t dh_experts_step_workspace_bytes(const dh_experts* spec);
+int dh_experts_step(const dh_experts* spec, float* d_x, void* d_workspace);
+/* T rows: d_h their normed rows [T][K] in the operand type (DH_BF16 or DH_F32), d_x the residual rows. */
+size_t dh_experts_prefill_workspace_bytes(const dh_experts* spec, int operand, int T);
+int dh_experts_prefill(const dh_experts* spec, const void* d_h, int operand, float* d_x, int ld_x, void* d_workspace, int T);
 
 /* ---- normalisation / rotary / KV ---- */
 
