@@ -13,6 +13,7 @@ through the C ABI, one 4-byte token readback per step.  Prints ONE JSON line wit
 
     python bench.py [--gpus 1] [--steps K] [--warmup W]
     python bench.py --design zepavik [--sizes 1024,2048,4096]     # that design beside the Q4_K decoder at equal size
+    python bench.py --design gusolorn [--sizes 1024,2048,4096]    # that design beside Zepavik at equal size
 """
 import argparse
 import ctypes
@@ -173,8 +174,8 @@ def main():
     ap.add_argument("--copy-calibration", action="store_true",
                     help="also run three f32->f16 casts of 16 Mi elements (64 MiB read, 32 MiB written): a "
                          "streaming kernel of known traffic to scale rocprofv3 FETCH_SIZE / WRITE_SIZE with")
-    ap.add_argument("--design", choices=("zepavik",), default=None,
-                    help="measure this design's prefill, decode and kernels beside the Q4_K decoder instead")
+    ap.add_argument("--design", choices=("zepavik", "gusolorn"), default=None,
+                    help="measure this design's prefill, decode and kernels beside the closest decoder instead")
     ap.add_argument("--sizes", default="1024,2048,4096", help="with --design: widths to measure")
     args = ap.parse_args()
     if args.gpus != 1:
@@ -193,7 +194,7 @@ def main():
     if args.design:
         from doppler_amd import design_bench
         sizes = args.sizes.split(",")
-        res = design_bench.run(sizes, args.steps, args.warmup)
+        res = design_bench.run(args.design, sizes, args.steps, args.warmup)
         last = res[sizes[-1]]
         print(json.dumps({"metric": "decode tokens/sec, %s at width %s, 1 GPU" % (args.design, sizes[-1]),
                           "value": last[args.design]["decode_tokens_per_s"], "unit": "tokens/s", "n_gpus": 1, "steps": args.steps,

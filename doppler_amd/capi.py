@@ -139,6 +139,7 @@ SIGNATURES = {
     "dh_dense_matmul": (_I, [_P, _I, _I, _P, _I, _I, _I, _I, _F, _P, _P, _P, _I, _I, _P, _I, _I, _I]),
     "dh_dense_matmul_scaled": (_I, [_P, _I, _I, _P, _I, _I, _I, _I, _F, _P, _P, _P, _P, _I, _I, _P, _I, _I, _I]),
     "dh_dense_gemv_scaled": (_I, [_P, _P, _I, _F, _P, _I, _I, _I, _F, _P, _P, _P, _P, _I, _P, _I]),
+    "dh_dense_gemv_heads": (_I, [_P, _P, _P, _I, _I, _I, _F, _P, _I, _I, _I, _P, _P, _P]),
     "dh_dense_gemv": (_I, [_P, _P, _I, _F, _P, _I, _I, _I, _F, _P, _P, _P, _I, _P, _I]),
     "dh_dense_lmhead_argmax": (_I, [_P, _P, _I, _F, _P, _I, _I, _I, _F, _P, _P, _I, _P]),
     "dh_embed_sum": (_I, [_P, _I, _P, _P, _I, _P, _I64, _I64, _I64, _P, _I, _P, _I, _I, _I, _I, _P]),

@@ -56,6 +56,9 @@ struct GemmArgs {
   dh::ExpertRows rows;    // GROUPED and GLU forms
 };
 
+// Second outputs a kernel is compiled for: none, one activation, or whatever the arguments say.
+constexpr int kNoSecond = -2, kAnyAct = -3;
+
 __device__ __forceinline__ void put_c2(const GemmArgs& a, int64_t at, float v) {
   if (a.c2_dtype == DH_BF16) static_cast<uint16_t*>(a.C2)[at] = dh::f32_to_bf16_bits(v);
   else if (a.c2_dtype == DH_F16) static_cast<_Float16*>(a.C2)[at] = (_Float16)v;
@@ -101,6 +104,7 @@ __device__ __forceinline__ int64_t source_row(const GemmArgs& a, const TilePlace
 }
 
 // One 32 x 32 accumulator tile: lane l holds column l & 31 and rows 8 (i / 4) + 4 (l >> 5) + i % 4.
+template <int ACT>
 __device__ __forceinline__ void store_tile(const GemmArgs& a, const TilePlace& p, const f32x16_t& acc, int m0, int n0, int lane) {
   const int n = n0 + (lane & 31);
   if (n >= a.N) return;
@@ -114,10 +118,35 @@ __device__ __forceinline__ void store_tile(const GemmArgs& a, const TilePlace& p
     }
     return;
   }
+  if (ACT == kNoSecond || n < a.n_first) {
+    const float scale = a.col_scale ? a.col_scale[n] : 1.f, bias = (a.bias ? a.bias[n] : 0.f) * scale, alpha = a.alpha * scale;
+    float* c = a.C + (int64_t)p.base * a.ldc + n;
+    if (a.residual) {
+      // every read in front of the first write: the residual may be the output itself
+      const float* res = a.residual + (int64_t)p.base * a.ldc + n;
+      float r[16];
 #pragma unroll
-  for (int i = 0; i < 16; i++) {
-    const int m = mb + 8 * (i >> 2) + (i & 3);
-    if (m < p.rows) put(a, p.base + m, n, acc[i]);
+      for (int i = 0; i < 16; i++) r[i] = res[(int64_t)min(mb + 8 * (i >> 2) + (i & 3), p.rows - 1) * a.ldc];
+#pragma unroll
+      for (int i = 0; i < 16; i++) {
+        const int m = mb + 8 * (i >> 2) + (i & 3);
+        if (m < p.rows) c[(int64_t)m * a.ldc] = fmaf(acc[i], alpha, bias) + r[i];
+      }
+    } else {
+#pragma unroll
+      for (int i = 0; i < 16; i++) {
+        const int m = mb + 8 * (i >> 2) + (i & 3);
+        if (m < p.rows) c[(int64_t)m * a.ldc] = fmaf(acc[i], alpha, bias);
+      }
+    }
+  } else {
+    const int64_t at = (int64_t)p.base * a.ldc2 + (n - a.n_first);
+    const int act = ACT == kAnyAct ? a.act : ACT;
+#pragma unroll
+    for (int i = 0; i < 16; i++) {
+      const int m = mb + 8 * (i >> 2) + (i & 3);
+      if (m < p.rows) put_c2(a, at + (int64_t)m * a.ldc2, dh::activate(acc[i] * a.alpha, act));
+    }
   }
 }
 // The same for a gate tile and the up tile beside it (first weight row n0 of the gate block).
@@ -138,8 +167,8 @@ __device__ __forceinline__ void store_glu(const GemmArgs& a, const TilePlace& p,
 }
 
 // WM x WN waves; a wave computes TM x TN accumulator tiles of 32 x 32.
-template <int WM, int WN, int TM, int TN, bool F16 = false, bool GROUPED = false, bool GLU = false>
-__global__ __launch_bounds__(64 * WM * WN) void gemm_16bit_kernel(const GemmArgs a) {
+template <int WM, int WN, int TM, int TN, bool F16, int ACT, bool GROUPED = false, bool GLU = false>
+__global__ __launch_bounds__(64 * WM * WN, TM * TN >= 4 ? 2 : TM * TN == 2 ? 3 : 4) void gemm_16bit_kernel(const GemmArgs a) {
   static_assert(!GLU || TN == 2, "a wave's two tiles are the gate and the up value");
   constexpr int BM = 32 * WM * TM, BN = 32 * WN * TN, THREADS = 64 * WM * WN;
   constexpr int PA = BM * 8 / THREADS, PB = BN * 8 / THREADS;      // 16-byte pieces per thread and tile
@@ -236,7 +265,7 @@ __global__ __launch_bounds__(64 * WM * WN) void gemm_16bit_kernel(const GemmArgs
       store_glu(a, place, acc[i][0], acc[i][1], m0 + 32 * (wm * TM + i), n0 + 32 * wn * TN, lane);
     } else {
 #pragma unroll
-      for (int j = 0; j < TN; j++) store_tile(a, place, acc[i][j], m0 + 32 * (wm * TM + i), n0 + 32 * (wn * TN + j), lane);
+      for (int j = 0; j < TN; j++) store_tile<ACT>(a, place, acc[i][j], m0 + 32 * (wm * TM + i), n0 + 32 * (wn * TN + j), lane);
     }
   }
 }
@@ -317,7 +346,7 @@ __global__ __launch_bounds__(256) void gemm_f32_kernel(const GemmArgs a) {
     store_glu(a, place, acc[0], acc[1], m0 + 32 * wm, n0 + 32 * wn * TN, lane);
   } else {
 #pragma unroll
-    for (int j = 0; j < TN; j++) store_tile(a, place, acc[j], m0 + 32 * wm, n0 + 32 * (wn * TN + j), lane);
+    for (int j = 0; j < TN; j++) store_tile<kAnyAct>(a, place, acc[j], m0 + 32 * wm, n0 + 32 * (wn * TN + j), lane);
   }
 }
 
@@ -331,7 +360,7 @@ __global__ __launch_bounds__(256) void gemm_reduce_kernel(const GemmArgs a, int 
   }
 }
 
-template <int WM, int WN, int TM, int TN, bool F16>
+template <int WM, int WN, int TM, int TN, bool F16, int ACT>
 int launch_16bit(const char* op, GemmArgs a, int slices) {
   a.tiles_m = (int)dh::ceil_div(a.M, 32 * WM * TM);
   a.tiles_n = (int)dh::ceil_div(a.N, 32 * WN * TN);
@@ -342,7 +371,7 @@ int launch_16bit(const char* op, GemmArgs a, int slices) {
     size_t bytes = 0;
     a.parts = dh::splitk_workspace(&bytes);
   }
-  hipLaunchKernelGGL((gemm_16bit_kernel<WM, WN, TM, TN, F16>), dim3(a.tiles_m * a.tiles_n, slices), dim3(64 * WM * WN), 0, dh::stream(), a);
+  hipLaunchKernelGGL((gemm_16bit_kernel<WM, WN, TM, TN, F16, ACT>), dim3(a.tiles_m * a.tiles_n, slices), dim3(64 * WM * WN), 0, dh::stream(), a);
   DH_CHECK_LAUNCH(op);
   if (a.parts) {
     const unsigned grid = (unsigned)std::min<int64_t>(dh::ceil_div((int64_t)a.M * a.N, 256), 4096);
@@ -352,7 +381,18 @@ int launch_16bit(const char* op, GemmArgs a, int slices) {
   return 0;
 }
 
-// Expert products: rows_max bounds the rows over all groups (the table of row tiles has room for that many).
+template <int WM, int WN, int TM, int TN>
+int launch_tile(const char* op, const GemmArgs& a, bool f16, int slices) {
+  if (f16) return a.n_first == a.N ? launch_16bit<WM, WN, TM, TN, true, kNoSecond>(op, a, slices)
+                  : a.act == DH_ACT_NONE ? launch_16bit<WM, WN, TM, TN, true, DH_ACT_NONE>(op, a, slices)
+                                         : launch_16bit<WM, WN, TM, TN, true, kAnyAct>(op, a, slices);
+  if (a.n_first == a.N) return launch_16bit<WM, WN, TM, TN, false, kNoSecond>(op, a, slices);
+  if (a.act == DH_ACT_RELU2) return launch_16bit<WM, WN, TM, TN, false, DH_ACT_RELU2>(op, a, slices);
+  if (a.act == DH_ACT_GELU_ERF) return launch_16bit<WM, WN, TM, TN, false, DH_ACT_GELU_ERF>(op, a, slices);
+  return launch_16bit<WM, WN, TM, TN, false, kAnyAct>(op, a, slices);
+}
+
+// Expert products; the grouped ones launch as many row tiles as the table has room for.
 template <bool GROUPED, bool GLU>
 int launch_experts(const char* op, GemmArgs a, int a_dtype, int bm) {
   a.k_slice = a.K;
@@ -365,9 +405,9 @@ int launch_experts(const char* op, GemmArgs a, int a_dtype, int bm) {
     a.tiles_n = (int)dh::ceil_div(a.N, 128);
     if (!GROUPED) a.tiles_m = (int)dh::ceil_div(a.M, bm);
     if (bm == 128)
-      hipLaunchKernelGGL((gemm_16bit_kernel<2, 2, 2, 2, false, GROUPED, GLU>), dim3(a.tiles_m * a.tiles_n), dim3(256), 0, dh::stream(), a);
+      hipLaunchKernelGGL((gemm_16bit_kernel<2, 2, 2, 2, false, kNoSecond, GROUPED, GLU>), dim3(a.tiles_m * a.tiles_n), dim3(256), 0, dh::stream(), a);
     else
-      hipLaunchKernelGGL((gemm_16bit_kernel<2, 2, 1, 2, false, GROUPED, GLU>), dim3(a.tiles_m * a.tiles_n), dim3(256), 0, dh::stream(), a);
+      hipLaunchKernelGGL((gemm_16bit_kernel<2, 2, 1, 2, false, kNoSecond, GROUPED, GLU>), dim3(a.tiles_m * a.tiles_n), dim3(256), 0, dh::stream(), a);
   }
   DH_CHECK_LAUNCH(op);
   return 0;
@@ -455,6 +495,6 @@ extern "C" int dh_dense_matmul_scaled(const void* d_A, int a_dtype, int lda, con
   const int pick = env_tile ? env_tile : big_enough ? 128 : 64;
   const int64_t t = tiles(pick, pick);
   const int slices = env_slices ? (int)std::min<int64_t>(env_slices, most) : t >= cus ? 1 : (int)slices_for(t, pick == 128 ? 2 : 4);
-  if (a_dtype == DH_F16) return pick == 128 ? launch_16bit<2, 2, 2, 2, true>(op, a, slices) : launch_16bit<2, 2, 1, 1, true>(op, a, slices);
-  return pick == 128 ? launch_16bit<2, 2, 2, 2, false>(op, a, slices) : launch_16bit<2, 2, 1, 1, false>(op, a, slices);
+  const bool f16 = a_dtype == DH_F16;
+  return pick == 128 ? launch_tile<2, 2, 2, 2>(op, a, f16, slices) : launch_tile<2, 2, 1, 1>(op, a, f16, slices);
 }

@@ -8,6 +8,9 @@
 //
 // Outputs as in the multi-row product (dense_gemm.hip): columns below n_first with bias, column scale and residual, the rest
 // through an activation; or the argmax over all of them (output head).
+//
+// The HEADS form reads the raw outputs of a layer's heads instead: each head divided by its root mean square, weighted and
+// multiplied by the sigmoid of an output gate on its way into LDS.
 #include <algorithm>
 #include <cfloat>
 
@@ -19,6 +22,7 @@ namespace {
 using dh::Cand;
 
 constexpr int kMaxK = 32768;
+constexpr int kMaxHeads = 256;        // of the HEADS form
 
 struct GemvArgs {
   const float* x;
@@ -36,12 +40,14 @@ struct GemvArgs {
   int n_first;
   float* C2;
   int act;
+  const float* gate;          // HEADS form: one number per element; norm_weight has one too, eps is the heads'
+  int heads, head_padded, head_size;
   int iters;                  // row groups per wave
   float* part_val;            // argmax: per-workgroup candidates
   uint32_t* part_idx;
 };
 
-template <int R, int U, int WAVES, bool ARGMAX>
+template <int R, int U, int WAVES, bool ARGMAX, bool HEADS>
 __global__ __launch_bounds__(64 * WAVES) void gemv_kernel(const GemvArgs a) {
   extern __shared__ __align__(16) float4 planes[];      // [2][K / 8]
   __shared__ float red[WAVES];
@@ -70,7 +76,32 @@ __global__ __launch_bounds__(64 * WAVES) void gemv_kernel(const GemvArgs a) {
   load(0, cur);
 
   // ---- the activation row
-  {
+  if constexpr (HEADS) {
+    __shared__ float inv_s[kMaxHeads];
+    const int hp = a.head_padded >> 2;                    // 16-byte pieces of a head
+    for (int h = wave; h < a.heads; h += WAVES) {
+      const float4* xh = reinterpret_cast<const float4*>(a.x) + (int64_t)h * hp;
+      float ss = 0.f;
+      for (int i = lane; i < hp; i += 64) {
+        const float4 v = xh[i];
+        ss = fmaf(v.x, v.x, ss); ss = fmaf(v.y, v.y, ss); ss = fmaf(v.z, v.z, ss); ss = fmaf(v.w, v.w, ss);
+      }
+      ss = dh::wave_sum_uniform(ss);
+      if (lane == 0) inv_s[h] = 1.0f / sqrtf(ss / (float)a.head_size + a.eps);
+    }
+    __syncthreads();
+    for (int i = tid; i < (a.K >> 2); i += THREADS) {
+      float4 v = make_float4(0.f, 0.f, 0.f, 0.f);
+      if (i < a.heads * hp) {
+        v = reinterpret_cast<const float4*>(a.x)[i];
+        const float4 w = reinterpret_cast<const float4*>(a.norm_weight)[i], g = reinterpret_cast<const float4*>(a.gate)[i];
+        const float f = inv_s[i / hp];
+        v.x = v.x * f * w.x / (1.0f + expf(-g.x)); v.y = v.y * f * w.y / (1.0f + expf(-g.y));
+        v.z = v.z * f * w.z / (1.0f + expf(-g.z)); v.w = v.w * f * w.w / (1.0f + expf(-g.w));
+      }
+      planes[(i & 1) * np + (i >> 1)] = v;
+    }
+  } else {
     const float4* xg = reinterpret_cast<const float4*>(a.x);
     float inv = 1.f;
     if (a.norm_weight) {
@@ -159,9 +190,9 @@ __global__ __launch_bounds__(64 * WAVES) void gemv_kernel(const GemvArgs a) {
   }
 }
 
-template <int R, int U, int WAVES, bool ARGMAX>
+template <int R, int U, int WAVES, bool ARGMAX, bool HEADS>
 int launch(const char* op, GemvArgs a, int max_grid, int* parts) {
-  auto kern = gemv_kernel<R, U, WAVES, ARGMAX>;
+  auto kern = gemv_kernel<R, U, WAVES, ARGMAX, HEADS>;
   static bool attr_set = false;
   if (!attr_set) {
     DH_CHECK_HIP(op, hipFuncSetAttribute(reinterpret_cast<const void*>(kern), hipFuncAttributeMaxDynamicSharedMemorySize,
@@ -177,7 +208,7 @@ int launch(const char* op, GemvArgs a, int max_grid, int* parts) {
   return 0;
 }
 
-template <bool ARGMAX>
+template <bool ARGMAX, bool HEADS = false>
 int dispatch(const char* op, const GemvArgs& a, int* parts) {
   // workgroups that are resident at once share the activation row's preparation as widely as the LDS allows
   const int cus = dh::num_cus();
@@ -185,10 +216,10 @@ int dispatch(const char* op, const GemvArgs& a, int* parts) {
   const bool two = env_r ? env_r == 2 : a.K <= 4096 && (int64_t)a.N >= (int64_t)64 * cus;
   if (a.K <= 8192) {
     const int max_grid = ARGMAX ? std::min(4 * cus, dh::kMaxParts) : 4 * cus;
-    return two ? launch<2, 4, 4, ARGMAX>(op, a, max_grid, parts) : launch<1, 8, 4, ARGMAX>(op, a, max_grid, parts);
+    return two ? launch<2, 4, 4, ARGMAX, HEADS>(op, a, max_grid, parts) : launch<1, 8, 4, ARGMAX, HEADS>(op, a, max_grid, parts);
   }
   const int max_grid = a.K <= 16384 ? 2 * cus : cus;
-  return launch<1, 8, 8, ARGMAX>(op, a, std::min(max_grid, dh::kMaxParts), parts);
+  return launch<1, 8, 8, ARGMAX, HEADS>(op, a, std::min(max_grid, dh::kMaxParts), parts);
 }
 
 int check(const char* op, const float* x, const float* norm_weight, int hidden, float eps, const void* W, int ldw, int N, int K) {
@@ -235,6 +266,22 @@ int dh_dense_gemv_scaled(const float* d_x, const float* d_norm_weight, int hidde
   GemvArgs a = make_args(d_x, d_norm_weight, hidden, eps, d_W, ldw, N, K, alpha);
   a.bias = d_bias; a.col_scale = d_col_scale; a.residual = d_residual; a.C = d_C; a.n_first = n_first; a.C2 = d_C2; a.act = activation;
   return dispatch<false>(op, a, nullptr);
+}
+
+int dh_dense_gemv_heads(const float* d_x, const float* d_gate, const float* d_weight, int H, int padded, int size, float eps, const void* d_W,
+                        int ldw, int N, int K, const float* d_col_scale, const float* d_residual, float* d_C) {
+  const char* op = "dh_dense_gemv_heads";
+  DH_REQUIRE_INIT(op);
+  if (int rc = check(op, d_x, nullptr, 0, eps, d_W, ldw, N, K)) return rc;
+  if (H <= 0 || H > kMaxHeads || size <= 0 || padded < size || padded % 4 || (int64_t)H * padded > K)
+    return dh::fail(1, "[%s] %d heads (at most %d) of %d elements, %d apart, in a row of %d", op, H, kMaxHeads, size, padded, K);
+  if (!d_gate || !d_weight || !d_C) return dh::fail(1, "[%s] null pointer", op);
+  if ((reinterpret_cast<uintptr_t>(d_gate) | reinterpret_cast<uintptr_t>(d_weight)) & 15) return dh::fail(1, "[%s] gate and weight must be 16-byte aligned", op);
+  if (d_x == d_C) return dh::fail(1, "[%s] the output must not be the activation row", op);
+  GemvArgs a = make_args(d_x, d_weight, 0, eps, d_W, ldw, N, K, 1.f);
+  a.gate = d_gate; a.heads = H; a.head_padded = padded; a.head_size = size;
+  a.col_scale = d_col_scale; a.residual = d_residual; a.C = d_C;
+  return dispatch<false, true>(op, a, nullptr);
 }
 
 int dh_dense_lmhead_argmax(const float* d_x, const float* d_norm_weight, int hidden, float eps, const void* d_W, int ldw,

@@ -42,32 +42,41 @@ struct StepArgs {
 __device__ __forceinline__ float sigmoid_f(float z) { return 1.0f / (1.0f + expf(-z)); }
 
 // The top experts of a row of logits, by one wave: ids (and logits) in the order of their size, the lower id first among equals.
-// Lane l holds experts l, l + 64, ...
-__device__ __forceinline__ void choose(const float* z, int E, int top, int* ids, float* zs) {
+// Lane l holds experts l, l + 64, .., 64 SLOTS in all; the maximum is found by lane steps, its lowest holder from a ballot.
+template <int SLOTS>
+__device__ __forceinline__ void choose_upto(const float* z, int E, int top, int* ids, float* zs) {
   const int lane = threadIdx.x & 63;
-  float v[kMaxExperts / 64];
+  float v[SLOTS];
 #pragma unroll
-  for (int j = 0; j < kMaxExperts / 64; j++) v[j] = lane + 64 * j < E ? z[lane + 64 * j] : -INFINITY;
+  for (int j = 0; j < SLOTS; j++) v[j] = lane + 64 * j < E ? z[lane + 64 * j] : -INFINITY;
   for (int t = 0; t < top; t++) {
-    float best = -INFINITY;
-    int id = 0x7FFFFFFF;
+    float best = v[0];
 #pragma unroll
-    for (int j = 0; j < kMaxExperts / 64; j++)
-      if (64 * j < E && (v[j] > best || id == 0x7FFFFFFF) && v[j] != -INFINITY) { best = v[j]; id = lane + 64 * j; }
+    for (int j = 1; j < SLOTS; j++) best = fmaxf(best, v[j]);
     const float mx = dh::group_combine<1, 64>(best, dh::MaxOp());
-    // the lowest id among the lanes that hold the maximum
-    int mine = best == mx && id != 0x7FFFFFFF ? id : 0x7FFFFFFF;
+    int id = 0;                                          // logits that are not numbers: some expert, inside the tables
+    bool found = false;
 #pragma unroll
-    for (int off = 1; off < 64; off <<= 1) mine = min(mine, __shfl_xor(mine, off, 64));
-    mine = mine >= E ? 0 : mine;                         // logits that are not numbers: some expert, inside the tables
+    for (int j = 0; j < SLOTS; j++) {
+      const unsigned long long at = __builtin_amdgcn_ballot_w64(v[j] == mx && lane + 64 * j < E);
+      if (!found && at != 0) {
+        id = 64 * j + __builtin_ctzll(at);
+        found = true;
+      }
+    }
     if (lane == 0) {
-      ids[t] = mine;
-      zs[t] = z[mine];
+      ids[t] = id;
+      zs[t] = mx;
     }
 #pragma unroll
-    for (int j = 0; j < kMaxExperts / 64; j++)
-      if (lane + 64 * j == mine) v[j] = -INFINITY;
+    for (int j = 0; j < SLOTS; j++)
+      if (lane + 64 * j == id) v[j] = -INFINITY;
   }
+}
+__device__ __forceinline__ void choose(const float* z, int E, int top, int* ids, float* zs) {
+  if (E <= 64) choose_upto<1>(z, E, top, ids, zs);
+  else if (E <= 256) choose_upto<4>(z, E, top, ids, zs);
+  else choose_upto<kMaxExperts / 64>(z, E, top, ids, zs);
 }
 
 // A wave takes a gate and an up row at a time; the row sits in LDS as two planes of 16-byte pieces, as in the dense GEMV.
@@ -260,7 +269,15 @@ __global__ __launch_bounds__(1024) void experts_sort_kernel(const int* __restric
   const int tid = threadIdx.x;
   count[tid] = 0;
   __syncthreads();
-  for (int i = tid; i < n; i += 1024) atomicAdd(&count[ids[i]], 1);
+  constexpr int BATCH = 8;                               // reads in flight per thread
+  for (int i0 = tid; i0 < n; i0 += 1024 * BATCH) {
+    int id[BATCH];
+#pragma unroll
+    for (int k = 0; k < BATCH; k++) id[k] = i0 + 1024 * k < n ? ids[i0 + 1024 * k] : -1;
+#pragma unroll
+    for (int k = 0; k < BATCH; k++)
+      if (id[k] >= 0) atomicAdd(&count[id[k]], 1);
+  }
   __syncthreads();
   const int mine = count[tid], my_tiles = (mine + tile_rows - 1) / tile_rows;
   scan[tid] = mine;
@@ -283,11 +300,24 @@ __global__ __launch_bounds__(1024) void experts_sort_kernel(const int* __restric
   for (int k = used + tid; k < max_tiles; k += 1024) tiles[2 * k] = -1;
   count[tid] = first;                                    // next free place of the expert
   __syncthreads();
-  for (int i = tid; i < n; i += 1024) {
-    const int at = atomicAdd(&count[ids[i]], 1);         // any order inside a group: a row's results do not depend on its place
-    slot[i] = at;
-    row_token[at] = i / top;
-    row_weight[at] = weights[i];
+  for (int i0 = tid; i0 < n; i0 += 1024 * BATCH) {
+    int id[BATCH];
+    float w[BATCH];
+#pragma unroll
+    for (int k = 0; k < BATCH; k++) {
+      const int i = i0 + 1024 * k;
+      id[k] = i < n ? ids[i] : -1;
+      w[k] = i < n ? weights[i] : 0.f;
+    }
+#pragma unroll
+    for (int k = 0; k < BATCH; k++) {
+      const int i = i0 + 1024 * k;
+      if (id[k] < 0) continue;
+      const int at = atomicAdd(&count[id[k]], 1);        // any order inside a group: a row's results do not depend on its place
+      slot[i] = at;
+      row_token[at] = i / top;
+      row_weight[at] = w[k];
+    }
   }
 }
 

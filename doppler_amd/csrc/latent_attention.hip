@@ -29,6 +29,9 @@ using dh::u32x4_t;
 constexpr float kLog2e = 1.4426950408889634f;
 constexpr int kKeys = 64;            // keys per pass
 constexpr int kVRow = kKeys + 8;     // halves per transposed latent row in LDS
+// Word of a transposed row that holds a key pair: groups of four words trade places by row, so that lanes that write eight rows
+// apart meet different banks; a group (what a fragment read takes) stays whole.
+__device__ __forceinline__ int v_word(int row, int pair) { return (row * kVRow >> 1) + (pair ^ (4 * ((row >> 3) & 7))); }
 
 struct LatentArgs {
   float* rows;             // projection rows [T][ld_row]
@@ -95,21 +98,14 @@ __global__ __launch_bounds__(256) void latent_rows_kernel(const LatentArgs a) {
   if (a.dkv_off >= 0) write_cache_row<KV>(a, row + a.dkv_off, pos, red);
 }
 
-// Dot product of a bf16 row (pieces of eight elements) with a vector in LDS, L lanes per row; all of them get it.
-// LONG: more pieces than lanes.
-template <int L, bool LONG = false>
-__device__ __forceinline__ float row_dot(const uint16_t* w, const float* x, int pieces, int piece) {
-  float s = 0.f;
-  for (int p = piece; LONG ? p < pieces : p == piece; p += L) {
-    if (!LONG && p >= pieces) break;
-    const u32x4_t v = *reinterpret_cast<const u32x4_t*>(w + 8 * p);
-    const float4 xa = *reinterpret_cast<const float4*>(x + 8 * p), xb = *reinterpret_cast<const float4*>(x + 8 * p + 4);
-    s = fmaf(xa.x, dh::bf16_low(v[0]), s); s = fmaf(xa.y, dh::bf16_high(v[0]), s);
-    s = fmaf(xa.z, dh::bf16_low(v[1]), s); s = fmaf(xa.w, dh::bf16_high(v[1]), s);
-    s = fmaf(xb.x, dh::bf16_low(v[2]), s); s = fmaf(xb.y, dh::bf16_high(v[2]), s);
-    s = fmaf(xb.z, dh::bf16_low(v[3]), s); s = fmaf(xb.w, dh::bf16_high(v[3]), s);
-  }
-  return dh::group_combine<1, L>(s, dh::AddOp());
+// s + eight bf16 elements times a vector in LDS.
+__device__ __forceinline__ float piece_dot(const u32x4_t v, const float* x, float s) {
+  const float4 xa = *reinterpret_cast<const float4*>(x), xb = *reinterpret_cast<const float4*>(x + 4);
+  s = fmaf(xa.x, dh::bf16_low(v[0]), s); s = fmaf(xa.y, dh::bf16_high(v[0]), s);
+  s = fmaf(xa.z, dh::bf16_low(v[1]), s); s = fmaf(xa.w, dh::bf16_high(v[1]), s);
+  s = fmaf(xb.x, dh::bf16_low(v[2]), s); s = fmaf(xb.y, dh::bf16_high(v[2]), s);
+  s = fmaf(xb.z, dh::bf16_low(v[3]), s); s = fmaf(xb.w, dh::bf16_high(v[3]), s);
+  return s;
 }
 
 __device__ __forceinline__ void put_query(const LatentArgs& a, int64_t at, float v) {
@@ -126,11 +122,19 @@ template <typename KV, int L>
 __global__ __launch_bounds__(256) void latent_query_kernel(const LatentArgs a) {
   __shared__ __align__(16) float qs[512];
   __shared__ float red[4];
-  const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, h = blockIdx.y;
+  constexpr int ROWS = 64 / L, PASSES = 16 / ROWS;       // L lanes hold a row of D <= 8 L elements
+  const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, h = blockIdx.y, piece = lane % L;
   const int64_t pos = step_position(a);
   if (h == a.H) {
     if (blockIdx.x == 0 && a.dkv_off >= 0) write_cache_row<KV>(a, a.rows + a.dkv_off, pos, red);
     return;
+  }
+  u32x4_t w[PASSES];
+#pragma unroll
+  for (int pass = 0; pass < PASSES; pass++) {
+    const int row = 64 * blockIdx.x + (4 * pass + wave) * ROWS + lane / L;      // C is a multiple of 64
+    w[pass] = u32x4_t{0u, 0u, 0u, 0u};
+    if (8 * piece < a.D) w[pass] = *reinterpret_cast<const u32x4_t*>(a.uk_t + ((int64_t)h * a.C + row) * a.D + 8 * piece);
   }
   const float* q = a.rows + (int64_t)h * (a.D + a.R);
   const float f = a.scale * kLog2e;
@@ -144,13 +148,11 @@ __global__ __launch_bounds__(256) void latent_query_kernel(const LatentArgs a) {
     }
   }
   __syncthreads();
-  constexpr int ROWS = 64 / L;
 #pragma unroll
-  for (int pass = 0; pass < 16 / ROWS; pass++) {
-    const int r = (4 * pass + wave) * ROWS + lane / L;
-    const int row = 64 * blockIdx.x + r;                 // C is a multiple of 64
-    const float s = row_dot<L>(a.uk_t + ((int64_t)h * a.C + row) * a.D, qs, a.D >> 3, lane % L);
-    if (lane % L == 0) put_query(a, base + row, s);
+  for (int pass = 0; pass < PASSES; pass++) {
+    const int row = 64 * blockIdx.x + (4 * pass + wave) * ROWS + lane / L;
+    const float s = dh::group_combine<1, L>(8 * piece < a.D ? piece_dot(w[pass], qs + 8 * piece, 0.f) : 0.f, dh::AddOp());
+    if (piece == 0) put_query(a, base + row, s);
   }
 }
 
@@ -180,6 +182,33 @@ __global__ __launch_bounds__(256) void latent_mfma_kernel(const LatentArgs a) {
   const int ntiles = (kr.kend - kr.kbeg + kKeys - 1) / kKeys;
   const _Float16* cache = static_cast<const _Float16*>(a.cache);
   const int64_t residual = (int64_t)a.H * CR;
+  // latents to be transposed: key pairs 8 wave + 4 i + (lane >> 4), sixteen neighbouring pieces of a row per group of lanes
+  const int piece0 = lane & 15, pair0 = 8 * wave + (lane >> 4);
+  constexpr int NP = (NT + 1) / 2;                       // pieces per lane: 16 NP pieces hold C elements
+  constexpr int KF = 2 * NT + 2;                         // key fragments in registers: rotated parts of up to 64 elements
+  const int steps = CR >> 5;
+  u32x4_t v[NP][2][2];
+  f16x8_t kf[KF];
+  auto key_row = [&](int k0) { return cache + (int64_t)min(k0 + 16 * wave + head, kr.kend - 1) * CR + 8 * g; };
+  // a tile's latents by key pairs (to be transposed) and key fragments; keys past the end repeat the last one (their
+  // probabilities are zero)
+  auto load = [&](int k0) {
+    const _Float16* krow = key_row(k0);
+#pragma unroll
+    for (int s = 0; s < KF; s++)
+      if (s < steps) kf[s] = *reinterpret_cast<const f16x8_t*>(krow + 32 * s);
+#pragma unroll
+    for (int j = 0; j < NP; j++) {
+      const int col = 8 * (piece0 + 16 * j);
+      if (col >= a.C) continue;
+#pragma unroll
+      for (int i = 0; i < 2; i++)
+#pragma unroll
+        for (int s = 0; s < 2; s++)
+          v[j][i][s] = *reinterpret_cast<const u32x4_t*>(cache + (int64_t)min(k0 + 2 * (pair0 + 4 * i) + s, kr.kend - 1) * CR + col);
+    }
+  };
+  if (split < ntiles) load(kr.kbeg + split * kKeys);
   for (int i = tid; i < 16 * (CR >> 3); i += 256) {
     const int hh = i / (CR >> 3), p = i % (CR >> 3);
     u32x4_t hi = {0u, 0u, 0u, 0u}, lo = hi;
@@ -194,26 +223,18 @@ __global__ __launch_bounds__(256) void latent_mfma_kernel(const LatentArgs a) {
 #pragma unroll
   for (int t = 0; t < NT; t++) acc[t] = {0.f, 0.f, 0.f, 0.f};
   float m_run = -FLT_MAX, l_run = 0.f;
-  const int pair = tid & 31, vcol = tid >> 5;
   __syncthreads();
   for (int c = split; c < ntiles; c += kr.nsplit) {
     const int k0 = kr.kbeg + c * kKeys;
-    // latents of key pairs, to be transposed; keys past the end repeat the last one (their probabilities are zero)
-    u32x4_t v[NT][2];
-#pragma unroll
-    for (int j = 0; j < NT; j++) {
-      if (64 * j >= a.C) break;
-#pragma unroll
-      for (int s = 0; s < 2; s++)
-        v[j][s] = *reinterpret_cast<const u32x4_t*>(cache + (int64_t)min(k0 + 2 * pair + s, kr.kend - 1) * CR + 8 * (vcol + 8 * j));
-    }
     f32x4_t st = {0.f, 0.f, 0.f, 0.f};
-    const _Float16* krow = cache + (int64_t)min(k0 + 16 * wave + head, kr.kend - 1) * CR + 8 * g;
-    for (int s = 0; s < (CR >> 5); s++) {
-      const f16x8_t ka = *reinterpret_cast<const f16x8_t*>(krow + 32 * s);
+    auto score = [&](const f16x8_t& ka, int s) {
       st = __builtin_amdgcn_mfma_f32_16x16x32_f16(ka, *reinterpret_cast<const f16x8_t*>(q_hi + head * qrow + 32 * s + 8 * g), st, 0, 0, 0);
       st = __builtin_amdgcn_mfma_f32_16x16x32_f16(ka, *reinterpret_cast<const f16x8_t*>(q_lo + head * qrow + 32 * s + 8 * g), st, 0, 0, 0);
-    }
+    };
+#pragma unroll
+    for (int s = 0; s < KF; s++)
+      if (s < steps) score(kf[s], s);
+    for (int s = KF; s < steps; s++) score(*reinterpret_cast<const f16x8_t*>(key_row(k0) + 32 * s), s);
     // this lane: head `head`, keys k0 + 16 wave + 4 g + i
     float mx = -FLT_MAX;
 #pragma unroll
@@ -224,14 +245,18 @@ __global__ __launch_bounds__(256) void latent_mfma_kernel(const LatentArgs a) {
     mx = dh::group_combine<16, 64>(mx, dh::MaxOp());
     if (g == 0) m_lds[wave][head] = mx;
 #pragma unroll
-    for (int j = 0; j < NT; j++) {
-      if (64 * j >= a.C) break;
+    for (int j = 0; j < NP; j++) {
+      const int col = 8 * (piece0 + 16 * j);
+      if (col >= a.C) continue;
 #pragma unroll
-      for (int e = 0; e < 8; e++) {
-        const uint32_t word = __builtin_amdgcn_perm(v[j][1][e >> 1], v[j][0][e >> 1], (e & 1) ? 0x07060302u : 0x05040100u);
-        reinterpret_cast<uint32_t*>(v_lds)[((8 * (vcol + 8 * j) + e) * kVRow >> 1) + pair] = word;
-      }
+      for (int i = 0; i < 2; i++)
+#pragma unroll
+        for (int e = 0; e < 8; e++) {
+          const uint32_t word = __builtin_amdgcn_perm(v[j][i][1][e >> 1], v[j][i][0][e >> 1], (e & 1) ? 0x07060302u : 0x05040100u);
+          reinterpret_cast<uint32_t*>(v_lds)[v_word(col + e, pair0 + 4 * i)] = word;
+        }
     }
+    if (c + kr.nsplit < ntiles) load(k0 + kr.nsplit * kKeys);
     __syncthreads();
     const float m_new = fmaxf(m_run, fmaxf(fmaxf(m_lds[0][head], m_lds[1][head]), fmaxf(m_lds[2][head], m_lds[3][head])));
     const float alpha = __builtin_amdgcn_exp2f(m_run - m_new);
@@ -259,7 +284,7 @@ __global__ __launch_bounds__(256) void latent_mfma_kernel(const LatentArgs a) {
       acc[t] *= alpha;
 #pragma unroll
       for (int kb = 0; kb < 2; kb++) {
-        const f16x8_t va = *reinterpret_cast<const f16x8_t*>(v_lds + (16 * tile + head) * kVRow + 32 * kb + 8 * g);
+        const f16x8_t va = *reinterpret_cast<const f16x8_t*>(reinterpret_cast<const uint32_t*>(v_lds) + v_word(16 * tile + head, 16 * kb + 4 * g));
         acc[t] = __builtin_amdgcn_mfma_f32_16x16x32_f16(va, *reinterpret_cast<const f16x8_t*>(p_hi + head * kVRow + 32 * kb + 8 * g), acc[t], 0, 0, 0);
         acc[t] = __builtin_amdgcn_mfma_f32_16x16x32_f16(va, *reinterpret_cast<const f16x8_t*>(p_lo + head * kVRow + 32 * kb + 8 * g), acc[t], 0, 0, 0);
       }
@@ -336,48 +361,88 @@ __global__ __launch_bounds__(256) void latent_plain_kernel(const LatentArgs a) {
   }
 }
 
-// Grid = (slices of 32 value elements, heads).
+// Grid = (slices of 32 value elements, heads).  The slice's weights are requested first and travel while the splits are merged.
 template <int L, bool LONG>
 __global__ __launch_bounds__(256) void latent_value_kernel(const LatentArgs a) {
   extern __shared__ __align__(16) float fl[];            // [C] the head's latent, [splits] factors
-  __shared__ float red[4];
+  __shared__ float4 sums[256];
   float* o = fl;
   float* f = fl + a.C;
-  const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, h = blockIdx.y;
+  constexpr int ROWS = 64 / L, PASSES = 8 / ROWS;
+  const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, h = blockIdx.y, piece = lane % L;
+  auto weights = [&](int pass) {
+    const int row = 32 * blockIdx.x + (4 * pass + wave) * ROWS + lane / L;
+    return a.uv + ((int64_t)h * a.VD + min(row, a.VD - 1)) * a.C;
+  };
+  u32x4_t w[PASSES];
+#pragma unroll
+  for (int pass = 0; pass < PASSES; pass++) {
+    w[pass] = u32x4_t{0u, 0u, 0u, 0u};
+    if (8 * piece < a.C) w[pass] = *reinterpret_cast<const u32x4_t*>(weights(pass) + 8 * piece);
+  }
   const int nsplit = key_range(a).nsplit, stride = a.C + 4;
   const float* base = a.parts + (int64_t)h * a.nsplit * stride;
+  // four latent elements per thread, the splits dealt to the groups of C / 4 threads; the first ones of a thread are requested here
+  constexpr int AHEAD = 8;
+  const int cols = a.C >> 2, groups = LONG ? 1 : 256 / cols, group = LONG ? 0 : tid / cols, col = 4 * (LONG ? tid : tid % cols);
+  float4 part[AHEAD];
+  if (!LONG && group < groups) {
+#pragma unroll
+    for (int k = 0; k < AHEAD; k++)
+      if (group + groups * k < nsplit) part[k] = *reinterpret_cast<const float4*>(base + (int64_t)(group + groups * k) * stride + col);
+  }
+  // every wave finds the common maximum and denominator by itself
   float M = -FLT_MAX;
-  for (int s = tid; s < nsplit; s += 256) M = fmaxf(M, base[(int64_t)s * stride + a.C]);
+  for (int s = lane; s < nsplit; s += 64) M = fmaxf(M, base[(int64_t)s * stride + a.C]);
   M = dh::group_combine<1, 64>(M, dh::MaxOp());
-  if (lane == 0) red[wave] = M;
-  __syncthreads();
-  M = fmaxf(fmaxf(red[0], red[1]), fmaxf(red[2], red[3]));
-  __syncthreads();
   float den = 0.f;
-  for (int s = tid; s < nsplit; s += 256) {
-    const float w = __builtin_amdgcn_exp2f(base[(int64_t)s * stride + a.C] - M);
-    f[s] = w;
-    den = fmaf(w, base[(int64_t)s * stride + a.C + 1], den);
+  for (int s = lane; s < nsplit; s += 64) {
+    const float e = __builtin_amdgcn_exp2f(base[(int64_t)s * stride + a.C] - M);
+    if (wave == 0) f[s] = e;
+    den = fmaf(e, base[(int64_t)s * stride + a.C + 1], den);
   }
   den = dh::wave_sum_uniform(den);
-  if (lane == 0) red[wave] = den;
-  __syncthreads();
-  den = red[0] + red[1] + red[2] + red[3];
   const float inv = den > 0.f ? 1.0f / den : 0.f;
-  for (int i = tid; i < a.C; i += 256) {
-    float v = 0.f;
-#pragma unroll 4
-    for (int s = 0; s < nsplit; s++) v = fmaf(f[s], base[(int64_t)s * stride + i], v);
-    o[i] = v * inv;
+  __syncthreads();
+  if (LONG) {
+    for (int i = tid; i < a.C; i += 256) {
+      float v = 0.f;
+#pragma unroll 8
+      for (int s = 0; s < nsplit; s++) v = fmaf(f[s], base[(int64_t)s * stride + i], v);
+      o[i] = v * inv;
+    }
+  } else {
+    float4 v = make_float4(0.f, 0.f, 0.f, 0.f);
+    auto add = [&](const float4& p, float e) {
+      v.x = fmaf(e, p.x, v.x); v.y = fmaf(e, p.y, v.y); v.z = fmaf(e, p.z, v.z); v.w = fmaf(e, p.w, v.w);
+    };
+    if (group < groups) {
+#pragma unroll
+      for (int k = 0; k < AHEAD; k++)
+        if (group + groups * k < nsplit) add(part[k], f[group + groups * k]);
+      for (int s = group + groups * AHEAD; s < nsplit; s += groups) add(*reinterpret_cast<const float4*>(base + (int64_t)s * stride + col), f[s]);
+      sums[tid] = make_float4(v.x * inv, v.y * inv, v.z * inv, v.w * inv);
+    }
+    __syncthreads();
+    if (tid < cols) {
+      float4 t = sums[tid];
+      for (int k = 1; k < groups; k++) {
+        const float4 u = sums[tid + k * cols];
+        t.x += u.x; t.y += u.y; t.z += u.z; t.w += u.w;
+      }
+      *reinterpret_cast<float4*>(o + 4 * tid) = t;
+    }
   }
   __syncthreads();
-  constexpr int ROWS = 64 / L;
 #pragma unroll
-  for (int pass = 0; pass < 8 / ROWS; pass++) {
-    const int r = (4 * pass + wave) * ROWS + lane / L;
-    const int row = 32 * blockIdx.x + r;
-    const float s = row_dot<L, LONG>(a.uv + ((int64_t)h * a.VD + min(row, a.VD - 1)) * a.C, o, a.C >> 3, lane % L);
-    if (lane % L == 0 && row < a.VD) a.out[(int64_t)h * a.VD + row] = s;
+  for (int pass = 0; pass < PASSES; pass++) {
+    const int row = 32 * blockIdx.x + (4 * pass + wave) * ROWS + lane / L;
+    float s = 8 * piece < a.C ? piece_dot(w[pass], o + 8 * piece, 0.f) : 0.f;
+    if (LONG) {
+      for (int p = piece + L; p < (a.C >> 3); p += L) s = piece_dot(*reinterpret_cast<const u32x4_t*>(weights(pass) + 8 * p), o + 8 * p, s);
+    }
+    s = dh::group_combine<1, L>(s, dh::AddOp());
+    if (piece == 0 && row < a.VD) a.out[(int64_t)h * a.VD + row] = s;
   }
 }
 

@@ -14,8 +14,10 @@
 // masked product inside it:
 //
 //   mlstm_gates_kernel     F, i, m of every token; one workgroup per head
-//   mlstm_states_kernel    the state in front of every chunk; a workgroup owns a 64 x 64 tile of one head's state and walks the
-//                          chunks:  S <- e^(F_end - F_start + m_start - m_end) S + sum_s e^(F_end - F_s + i_s - m_end) k_s v_s^T
+//   mlstm_chunks_kernel    what every chunk adds to the state behind it, sum_s e^(F_end - F_s + i_s - m_end) k_s v_s^T: independent of
+//                          one another, because m is known
+//   mlstm_scan_kernel      the state in front of every chunk, S_(c+1) = e^(F_end - F_start + m_start - m_end) S_c + what chunk c adds,
+//                          element by element and in place
 //   mlstm_outputs_kernel   o of (chunk, head, value columns): Q K^T and Q S in one walk over dim, decay mask, then (Q K^T) V
 //
 // on the 32-bit matrix-core instruction v_mfma_f32_32x32x2_f32.  head_norm_gate_kernel then divides every head's output by its root
@@ -50,8 +52,9 @@ struct MemArgs {
   float* i;
   float* mt;               // m after every token
   float* mc;               // [H][chunks + 1] m in front of every chunk, and at the end
-  float* Sc;               // [chunks][H][DP][VP]
-  float* nc;               // [chunks][H][DP]
+  float* keep;             // [H][chunks] what a chunk leaves of the state in front of it
+  float* Sc;               // [chunks + 1][H][DP][VP]
+  float* nc;               // [chunks + 1][H][DP]
 };
 
 __device__ __forceinline__ float log_input_gate(const MemArgs& a, float z) { return a.gate_cap * tanhf(z / a.gate_cap); }
@@ -167,86 +170,97 @@ __global__ __launch_bounds__(1024) void mlstm_gates_kernel(const MemArgs a) {
       a.m[((a.pos + a.T) & 1) * a.H + h] = (float)m;
     }
   }
+  __syncthreads();
+  for (int c = tid; c < a.chunks; c += 1024) {
+    const double start = c > 0 ? F[c * kChunk - 1] : 0.0, end = F[min((c + 1) * kChunk, a.T) - 1];
+    a.keep[(int64_t)h * a.chunks + c] = expf((float)(end - start + (double)mc[c] - (double)mc[c + 1]));
+  }
 }
 
-// Grid = (64 x 64 tiles of a head's state, heads); wave w: rows 32 (w >> 1), columns 32 (w & 1) of the tile.
-__global__ __launch_bounds__(256) void mlstm_states_kernel(const MemArgs a) {
+// Grid = (64 x 64 tiles of a head's state, heads, chunks); wave w: rows 32 (w >> 1), columns 32 (w & 1) of the tile.
+__global__ __launch_bounds__(256) void mlstm_chunks_kernel(const MemArgs a) {
   constexpr int ROW = 64 + 4;
   __shared__ __align__(16) float ks[kChunk * ROW];     // weighted keys [token][dim]
   __shared__ __align__(16) float vs[kChunk * ROW];     // values [token][column]
-  __shared__ float ws[kChunk];
-  const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, h = blockIdx.y;
+  const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, h = blockIdx.y, c = blockIdx.z;
   const int tiles_v = (a.VP + 63) / 64, d0 = 64 * (blockIdx.x / tiles_v), v0 = 64 * (blockIdx.x % tiles_v);
-  const int wd = d0 + 32 * (wave >> 1), wv = v0 + 32 * (wave & 1);
-  const bool live = wd < a.DP && wv < a.VP;            // wave-uniform (sizes are multiples of 32)
   const double* F = a.F + (int64_t)h * a.T;
-  const float* li = a.i + (int64_t)h * a.T;
-  const float* mc = a.mc + (int64_t)h * (a.chunks + 1);
-  float* S = a.S + (int64_t)h * a.DP * a.VP;
-  // accumulator element e of a lane: state row wd + 8 (e / 4) + 4 (lane >> 5) + e % 4, column wv + (lane & 31)
-  const int64_t at0 = (int64_t)(wd + 4 * (lane >> 5)) * a.VP + wv + (lane & 31);
-  f32x16_t acc;
-#pragma unroll
-  for (int e = 0; e < 16; e++) acc[e] = live && a.pos > 0 ? S[at0 + (int64_t)(8 * (e >> 2) + (e & 3)) * a.VP] : 0.f;
-  const bool owns_n = v0 == 0 && tid < 64 && d0 + tid < a.DP;
-  float n = owns_n && a.pos > 0 ? a.n[((int64_t)(a.pos & 1) * a.H + h) * a.DP + d0 + tid] : 0.f;
-
+  const int first = c * kChunk, count = min(kChunk, a.T - first);
+  const double F_end = F[first + count - 1];
+  const float m_end = a.mc[(int64_t)h * (a.chunks + 1) + c + 1];
   f32x4_t kr[4], vr[4];
-  auto load = [&](int c) {
+  float w[4];
 #pragma unroll
-    for (int r = 0; r < 4; r++) {
-      const int p = tid + 256 * r, tok = min(c * kChunk + (p >> 4), a.T - 1), x = 4 * (p & 15);
-      const float* row = a.rows + (int64_t)tok * a.ld_row;
-      kr[r] = vr[r] = f32x4_t{0.f, 0.f, 0.f, 0.f};
-      if (d0 + x < a.DP) kr[r] = *reinterpret_cast<const f32x4_t*>(row + a.k_off + (int64_t)h * a.DP + d0 + x);
-      if (v0 + x < a.VP) vr[r] = *reinterpret_cast<const f32x4_t*>(row + a.v_off + (int64_t)h * a.VP + v0 + x);
-    }
-  };
-  load(0);
-  for (int c = 0; c < a.chunks; c++) {
-    const int first = c * kChunk, count = min(kChunk, a.T - first);
-    const double F_end = F[first + count - 1], F_start = first > 0 ? F[first - 1] : 0.0;
-    const float m_start = mc[c], m_end = mc[c + 1];
-    if (live) {
-      float* Sc = a.Sc + ((int64_t)c * a.H + h) * a.DP * a.VP;
+  for (int r = 0; r < 4; r++) {
+    const int p = tid + 256 * r, tok = first + min(p >> 4, count - 1), x = 4 * (p & 15);
+    const float* row = a.rows + (int64_t)tok * a.ld_row;
+    kr[r] = vr[r] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+    if (d0 + x < a.DP) kr[r] = *reinterpret_cast<const f32x4_t*>(row + a.k_off + (int64_t)h * a.DP + d0 + x);
+    if (v0 + x < a.VP) vr[r] = *reinterpret_cast<const f32x4_t*>(row + a.v_off + (int64_t)h * a.VP + v0 + x);
+    w[r] = (p >> 4) < count ? expf((float)(F_end - F[tok] + (double)a.i[(int64_t)h * a.T + tok] - (double)m_end)) : 0.f;
+  }
 #pragma unroll
-      for (int e = 0; e < 16; e++) Sc[at0 + (int64_t)(8 * (e >> 2) + (e & 3)) * a.VP] = acc[e];
-    }
-    if (owns_n) a.nc[((int64_t)c * a.H + h) * a.DP + d0 + tid] = n;
-    if (tid < kChunk) ws[tid] = tid < count ? expf((float)(F_end - F[first + tid] + (double)li[first + tid] - (double)m_end)) : 0.f;
-    __syncthreads();                                   // weights are there, the previous chunk has been consumed
+  for (int r = 0; r < 4; r++) {
+    const int p = tid + 256 * r, tok = p >> 4, x = 4 * (p & 15);
+    kr[r] *= w[r];
+    *reinterpret_cast<f32x4_t*>(&ks[tok * ROW + x]) = kr[r];
+    *reinterpret_cast<f32x4_t*>(&vs[tok * ROW + x]) = vr[r];
+  }
+  __syncthreads();
+  const int wd = 32 * (wave >> 1), wv = 32 * (wave & 1);
+  if (d0 + wd < a.DP && v0 + wv < a.VP) {              // wave-uniform (sizes are multiples of 32)
+    f32x16_t acc;
 #pragma unroll
-    for (int r = 0; r < 4; r++) {
-      const int p = tid + 256 * r, tok = p >> 4, x = 4 * (p & 15);
-      const float w = ws[tok];
-      f32x4_t kw = kr[r];
-      kw *= w;
-      *reinterpret_cast<f32x4_t*>(&ks[tok * ROW + x]) = kw;
-      *reinterpret_cast<f32x4_t*>(&vs[tok * ROW + x]) = vr[r];
-    }
-    __syncthreads();
-    if (c + 1 < a.chunks) load(c + 1);
-    const float keep = expf((float)(F_end - F_start + (double)m_start - (double)m_end));
-#pragma unroll
-    for (int e = 0; e < 16; e++) acc[e] *= keep;
+    for (int e = 0; e < 16; e++) acc[e] = 0.f;
 #pragma unroll 8
     for (int j = 0; j < kChunk / 2; j++) {
       const int tok = 2 * j + (lane >> 5);
-      acc = __builtin_amdgcn_mfma_f32_32x32x2f32(ks[tok * ROW + 32 * (wave >> 1) + (lane & 31)], vs[tok * ROW + 32 * (wave & 1) + (lane & 31)], acc, 0, 0, 0);
+      acc = __builtin_amdgcn_mfma_f32_32x32x2f32(ks[tok * ROW + wd + (lane & 31)], vs[tok * ROW + wv + (lane & 31)], acc, 0, 0, 0);
     }
-    if (owns_n) {
-      float s = 0.f;
-#pragma unroll 8
-      for (int t = 0; t < kChunk; t++) s += ks[t * ROW + tid];
-      n = fmaf(keep, n, s);
-    }
-    __syncthreads();
-  }
-  if (live) {
+    // accumulator element e of a lane: state row 8 (e / 4) + 4 (lane >> 5) + e % 4, column lane & 31
+    float* U = a.Sc + ((int64_t)(c + 1) * a.H + h) * a.DP * a.VP + (int64_t)(d0 + wd + 4 * (lane >> 5)) * a.VP + v0 + wv + (lane & 31);
 #pragma unroll
-    for (int e = 0; e < 16; e++) S[at0 + (int64_t)(8 * (e >> 2) + (e & 3)) * a.VP] = acc[e];
+    for (int e = 0; e < 16; e++) U[(int64_t)(8 * (e >> 2) + (e & 3)) * a.VP] = acc[e];
   }
-  if (owns_n) a.n[((int64_t)((a.pos + a.T) & 1) * a.H + h) * a.DP + d0 + tid] = n;
+  if (v0 == 0 && tid < 64 && d0 + tid < a.DP) {
+    float s = 0.f;
+#pragma unroll 8
+    for (int t = 0; t < kChunk; t++) s += ks[t * ROW + tid];
+    a.nc[((int64_t)(c + 1) * a.H + h) * a.DP + d0 + tid] = s;
+  }
+}
+
+// Grid = (groups of 1024 elements of a head's [S | n], heads), four per thread; slot 0 of Sc and nc is filled here.
+__global__ __launch_bounds__(256) void mlstm_scan_kernel(const MemArgs a) {
+  constexpr int AHEAD = 16;
+  const int h = blockIdx.y, size = a.DP * a.VP;
+  const int64_t i = 4 * ((int64_t)blockIdx.x * 256 + threadIdx.x);
+  if (i >= size + a.DP) return;
+  const bool is_n = i >= size;
+  const int64_t stride = is_n ? (int64_t)a.H * a.DP : (int64_t)a.H * size;
+  float* at = is_n ? a.nc + (int64_t)h * a.DP + (i - size) : a.Sc + (int64_t)h * size + i;
+  const int64_t slots = (int64_t)a.H * a.DP;
+  const float* from = is_n ? a.n + (a.pos & 1) * slots + (int64_t)h * a.DP + (i - size) : a.S + (int64_t)h * size + i;
+  float* to = is_n ? a.n + ((a.pos + a.T) & 1) * slots + (int64_t)h * a.DP + (i - size) : a.S + (int64_t)h * size + i;
+  const float* keep = a.keep + (int64_t)h * a.chunks;
+  f32x4_t s = {0.f, 0.f, 0.f, 0.f};
+  if (a.pos > 0) s = *reinterpret_cast<const f32x4_t*>(from);
+  *reinterpret_cast<f32x4_t*>(at) = s;
+  for (int c0 = 0; c0 < a.chunks; c0 += AHEAD) {
+    f32x4_t u[AHEAD];
+#pragma unroll
+    for (int k = 0; k < AHEAD; k++)
+      if (c0 + k < a.chunks) u[k] = *reinterpret_cast<const f32x4_t*>(at + (c0 + k + 1) * stride);
+#pragma unroll
+    for (int k = 0; k < AHEAD; k++) {
+      const int c = c0 + k;
+      if (c < a.chunks) {
+        s = s * keep[c] + u[k];
+        if (c + 1 < a.chunks) *reinterpret_cast<f32x4_t*>(at + (c + 1) * stride) = s;
+      }
+    }
+  }
+  *reinterpret_cast<f32x4_t*>(to) = s;
 }
 
 // Grid = (chunks, heads, groups of 64 TN value columns); wave w: tokens 32 (w >> 1), columns 32 TN (w & 1) + 0 .. 32 TN - 1.
@@ -482,8 +496,8 @@ int dh_mlstm_step(const dh_mlstm* spec, const float* d_row, void* d_state, float
 size_t dh_mlstm_prefill_workspace_bytes(const dh_mlstm* s, int T) {
   if (!s || T <= 0) return 256;
   const size_t chunks = (size_t)dh::ceil_div(T, kChunk), HT = (size_t)s->H * T;
-  return up256(HT * 8) + 2 * up256(HT * 4) + up256((size_t)s->H * (chunks + 1) * 4) + up256(chunks * s->H * s->DP * 4) +
-         up256(chunks * s->H * s->DP * s->VP * 4);
+  return up256(HT * 8) + 2 * up256(HT * 4) + 2 * up256((size_t)s->H * (chunks + 1) * 4) + up256((chunks + 1) * s->H * s->DP * 4) +
+         up256((chunks + 1) * s->H * s->DP * s->VP * 4);
 }
 
 int dh_mlstm_prefill(const dh_mlstm* spec, const float* d_rows, void* d_state, void* d_workspace, float* d_out, int ld_out, int T,
@@ -504,12 +518,17 @@ int dh_mlstm_prefill(const dh_mlstm* spec, const float* d_rows, void* d_state, v
   a.i = reinterpret_cast<float*>(take(HT * 4));
   a.mt = reinterpret_cast<float*>(take(HT * 4));
   a.mc = reinterpret_cast<float*>(take((size_t)spec->H * (a.chunks + 1) * 4));
-  a.nc = reinterpret_cast<float*>(take((size_t)a.chunks * spec->H * spec->DP * 4));
-  a.Sc = reinterpret_cast<float*>(take((size_t)a.chunks * spec->H * spec->DP * spec->VP * 4));
+  a.keep = reinterpret_cast<float*>(take((size_t)spec->H * (a.chunks + 1) * 4));
+  a.nc = reinterpret_cast<float*>(take((size_t)(a.chunks + 1) * spec->H * spec->DP * 4));
+  a.Sc = reinterpret_cast<float*>(take((size_t)(a.chunks + 1) * spec->H * spec->DP * spec->VP * 4));
   hipLaunchKernelGGL(mlstm_gates_kernel, dim3(spec->H), dim3(1024), 0, dh::stream(), a);
   DH_CHECK_LAUNCH(op);
   const int tiles = (int)(dh::ceil_div(spec->DP, 64) * dh::ceil_div(spec->VP, 64));
-  hipLaunchKernelGGL(mlstm_states_kernel, dim3(tiles, spec->H), dim3(256), 0, dh::stream(), a);
+  // the grid's third dimension holds at most 65535 chunks
+  if (a.chunks > 65535) return dh::fail(1, "[%s] %d tokens are too many for one portion", op, T);
+  hipLaunchKernelGGL(mlstm_chunks_kernel, dim3(tiles, spec->H, a.chunks), dim3(256), 0, dh::stream(), a);
+  DH_CHECK_LAUNCH(op);
+  hipLaunchKernelGGL(mlstm_scan_kernel, dim3((unsigned)dh::ceil_div((int64_t)spec->DP * spec->VP + spec->DP, 1024), spec->H), dim3(256), 0, dh::stream(), a);
   DH_CHECK_LAUNCH(op);
   // wide column groups repeat Q K^T less often; narrow ones where those would not fill the device
   const bool wide = spec->VP > 64 && (int64_t)a.chunks * spec->H * dh::ceil_div(spec->VP, 128) >= dh::num_cus();

@@ -1,6 +1,7 @@
 """Throughput of a design beside the closest decoder the package serves, at sizes that resemble a real model's layers.
 
-Zepavik (dense bf16, parallel layers, windowed attention) against the Q4_K decoder with the same width, heads, feed-forward
+Gusolorn (sequential layers: latent attention with a dense feed-forward, two of matrix memory with experts, and again) against Zepavik
+with the same width, heads, layer count, window and active feed-forward width.  Zepavik (dense bf16, parallel layers, windowed attention) against the Q4_K decoder with the same width, heads, feed-forward
 width and layer count: prefill and decode tokens/s, and per kernel the share of its roofline (8 TB/s of HBM, 2.5
 PFLOP/s on the matrix cores).  Random weights; kernels cycle through more weights than the caches hold.
 """
@@ -9,12 +10,19 @@ import sys
 import time
 
 import numpy as np
+import torch
 
-HBM_GBPS, MFMA_TFLOPS = 8000.0, 2500.0
+HBM_GBPS, MFMA_TFLOPS, MFMA_F32_TFLOPS = 8000.0, 2500.0, 157.3
 SIZES = {
     "1024": dict(hidden=1024, heads=16, kv_heads=8, head_dim=64, ff=3072, layers=24),
     "2048": dict(hidden=2048, heads=16, kv_heads=8, head_dim=128, ff=6144, layers=12),
     "4096": dict(hidden=4096, heads=32, kv_heads=8, head_dim=128, ff=12288, layers=6),
+}
+# what the second design's mixers add to a size: latent (dim, rotated, value, rank), memory (heads, dim, value), experts (count, top)
+MIXED = {
+    "1024": dict(latent=(64, 32, 64, 256), memory=(4, 128, 256), experts=(16, 4)),
+    "2048": dict(latent=(128, 64, 128, 512), memory=(4, 256, 512), experts=(16, 4)),
+    "4096": dict(latent=(128, 64, 128, 512), memory=(8, 256, 512), experts=(16, 4)),
 }
 VOCAB, WINDOW, PROMPT = 32000, 1024, 2048
 
@@ -29,6 +37,24 @@ def zepavik_config(s, max_seq):
     return dict(hidden=s["hidden"], vocab=VOCAB, eps=1e-5, logit_scale=1.0, max_positions=max_seq,
                 bigram=dict(buckets=4096, mul_prev=31, mul_cur=7),
                 layers=[dict(mixer=dict(mixer), mlp=dict(ff=s["ff"], activation="relu2")) for _ in range(s["layers"])])
+
+
+def gusolorn_config(s, mixed):
+    d, rot, e, rank = mixed["latent"]
+    H, md, me = mixed["memory"]
+    E, top = mixed["experts"]
+    latent = dict(type="latent_attention", heads=s["heads"], dim=d, rot_dim=rot, vdim=e, kv_rank=rank, window=WINDOW, scale=(d + rot) ** -0.5,
+                  rot_base=10000.0, kv_from=None)
+    memory = dict(type="mlstm", heads=H, dim=md, vdim=me, gate_cap=15.0)
+    experts = dict(type="experts", experts=E, top=top, ff=s["ff"] // 2 // top, limit=7.0, shared=dict(ff=s["ff"] // 2, limit=7.0))
+    layers = []
+    for i in range(s["layers"]):
+        if i % 3 == 0:      # every second latent layer borrows the rows of the one before it
+            layers.append(dict(sequential=True, mixer=dict(latent, kv_from=i - 3 if i % 6 == 3 else None),
+                               mlp=dict(type="dense", ff=s["ff"], activation="gelu_erf")))
+        else:
+            layers.append(dict(sequential=True, mixer=dict(memory), mlp=dict(experts)))
+    return dict(hidden=s["hidden"], vocab=VOCAB, eps=1e-6, logit_scale=1.0, max_positions=0, bigram=None, layers=layers)
 
 
 def q4k_config(s, max_seq):
@@ -83,12 +109,24 @@ def _throughput(dec, prompt, steps, warmup):
     return prefill, decode
 
 
-def _entry(name, us, nbytes=None, flops=None):
+def _replayed(dec, pos, steps):
+    """Decode tokens/s of the captured step, one replay and one token readback per token."""
+    tok = dec.step_graph(1, pos)
+    dec.L.dh_sync()
+    t0 = time.perf_counter()
+    for k in range(steps):
+        tok = dec.step_graph(tok, pos + 1 + k)
+    rate = steps / (time.perf_counter() - t0)
+    dec.release_graph()
+    return rate
+
+
+def _entry(name, us, nbytes=None, flops=None, peak=MFMA_TFLOPS):
     e = dict(kernel=name, us=round(us, 2))
     if nbytes is not None:
         e.update(gb_per_s=round(nbytes / us / 1e3, 1), hbm_frac=round(nbytes / us / 1e3 / HBM_GBPS, 4))
     else:
-        e.update(tflop_per_s=round(flops / us / 1e6, 1), mfma_frac=round(flops / us / 1e6 / MFMA_TFLOPS, 4))
+        e.update(tflop_per_s=round(flops / us / 1e6, 1), mfma_frac=round(flops / us / 1e6 / peak, 4))
     return e
 
 
@@ -138,6 +176,82 @@ def zepavik_kernels(dec, s, T):
     return out
 
 
+def gusolorn_kernels(dec, s, T):
+    from . import capi, sublayers as sl
+    L, ck, c = dec.L, capi.check, dec.cfg
+    t, pos, Hd = _Timer(L), PROMPT + 8, c["hidden"]
+    kinds = lambda kind: [p for layer in dec.layers for p in layer.parts if isinstance(p, kind)]
+    latent, memory, dense, experts = (kinds(k) for k in (sl.LatentAttention, sl.MatrixMemory, sl.DenseFF, sl.ExpertsFF))
+    out, f32, x = [], torch.float32, dec.x.data_ptr()
+    row = lambda p: dec.scratch.rows("row", p.ld if hasattr(p, "ld") else p.n_in, 1, f32)
+    mixed = lambda p: dec.scratch.rows("mixed", p.k2, 1, f32)
+    px = dec._pf["x"].data_ptr()
+
+    def add(name, parts, f, nbytes=None, flops=None, peak=MFMA_TFLOPS):
+        us = t.us([(lambda p=p: f(p)) for p in parts])
+        out.append(_entry(name, us, nbytes=nbytes, flops=flops, peak=peak))
+    own = [p for p in latent if p.lender is None]
+    m = latent[0].m
+    H, d, rot, e, rank = m["heads"], m["dim"], m["rot_dim"], m["vdim"], m["kv_rank"]
+    n_in = H * (d + rot) + rank + rot
+    add("decode: latent, norm + q/latent", own, lambda p: p._gemv(x, True, p.w_in, p.n_in, p.kx, out=row(p)), nbytes=2.0 * n_in * Hd)
+    add("decode: latent attention, %d keys (with up projections)" % WINDOW, latent, lambda p: ck(L.dh_latent_decode(
+        p.ref, row(p), p.cache.data_ptr(), mixed(p), pos, None, dec.max_seq, dec.scratch.space("latent_decode", 1))),
+        nbytes=2.0 * (H * rank * (d + e) + WINDOW * (rank + rot)))
+    add("decode: latent, o + residual", latent, lambda p: p._gemv(mixed(p), False, p.w_out, Hd, p.k2, residual=True), nbytes=2.0 * Hd * H * e)
+    mm = memory[0].m
+    MH, md, me = mm["heads"], mm["dim"], mm["vdim"]
+    add("decode: memory, norm + q/k/v/gates", memory, lambda p: p._gemv(x, True, p.w_in, p.n_in, p.kx, bias=p.bias.data_ptr(), out=row(p)),
+        nbytes=2.0 * MH * (2 * md + 2 * me + 2) * Hd)
+    heads = lambda p: dec.scratch.rows("heads", p.o_width, 1, f32)
+    add("decode: memory, state step", memory, lambda p: ck(L.dh_mlstm_step(p.ref, row(p), p.memory.data_ptr(), heads(p), pos, None)),
+        nbytes=8.0 * MH * md * (me + 1))
+    add("decode: memory, head norm, gate, o + residual", memory, lambda p: p._out_step(heads(p), row(p)), nbytes=2.0 * Hd * MH * me)
+    ff = dense[0].ff
+    act = dec.scratch.rows("act", dense[0].ffp, 1, f32)
+    add("decode: dense ff, norm + up", dense, lambda p: p._gemv(x, True, p.up, p.ff, p.kx, act_out=act, act=p.act), nbytes=2.0 * ff * Hd)
+    add("decode: dense ff, down + residual", dense, lambda p: p._gemv(act, False, p.down, Hd, p.ffp, residual=True), nbytes=2.0 * ff * Hd)
+    add("decode: experts (router, up, down)", experts, lambda p: p.step(pos, None), nbytes=float(experts[0].step_bytes(0)))
+    us = t.us([lambda: dec._enqueue_head(x, 0, None)] * 4)
+    out.append(_entry("decode: norm + head + argmax (weights in cache where they fit)", us, nbytes=2.0 * c["vocab"] * Hd))
+
+    def in_rows(p):
+        normed = p._normed_rows(px, T)
+        ld = p.ld if hasattr(p, "ld") else p.n_in
+        ck(L.dh_dense_matmul(normed, dec.operand, p.kx, p.w_in.data_ptr(), p.kx, T, p.n_in, p.kx, 1.0, p.bias.data_ptr() if hasattr(p, "bias") else None,
+                             None, dec.scratch.rows("rows", ld, T, f32), ld, p.n_in, None, 0, 0, capi.ACT_NONE))
+    mixed_rows = lambda p: dec.scratch.rows("mixed_rows", p.k2, T, dec.operand_torch)
+    rows = lambda p: dec.scratch.rows("rows", p.ld if hasattr(p, "ld") else p.n_in, T, f32)
+    add("prefill: latent, norm, q/latent", own, in_rows, flops=2.0 * T * n_in * Hd)
+    add("prefill: latent, rotation + cache rows", own, lambda p: ck(L.dh_latent_rows(p.ref, rows(p), p.cache.data_ptr(), T, 0)),
+        nbytes=float(T * (8 * H * rot + 6 * (rank + rot))))
+    ws = dec.scratch.space("latent_prefill", L.dh_latent_prefill_workspace_bytes(latent[0].ref, T, 0))
+    pairs = _attn_flops(T, 1, 1, WINDOW) / 4
+    add("prefill: latent attention, window %d (with up projections)" % WINDOW, latent, lambda p: ck(L.dh_latent_prefill(
+        p.ref, rows(p), p.cache.data_ptr(), ws, mixed_rows(p), dec.operand, p.k2, T, 0)),
+        flops=2.0 * H * (pairs * (d + rot + e) + T * rank * (d + e)))
+    add("prefill: latent, o + residual", latent, lambda p: p._out_rows(mixed_rows(p), p.k2, p.w_out, px, T), flops=2.0 * T * Hd * H * e)
+    add("prefill: memory, norm, q/k/v/gates", memory, in_rows, flops=2.0 * T * Hd * MH * (2 * md + 2 * me + 2))
+    mws = dec.scratch.space("mlstm_prefill", L.dh_mlstm_prefill_workspace_bytes(memory[0].ref, T))
+    head_rows = lambda p: dec.scratch.rows("heads_rows", p.o_width, T, f32)
+    add("prefill: memory, chunks (32-bit products)", memory, lambda p: ck(L.dh_mlstm_prefill(p.ref, rows(p), p.memory.data_ptr(), mws, head_rows(p), p.o_width, T, 0)),
+        flops=2.0 * T * MH * (2 * md * me + 32 * (md + me)), peak=MFMA_F32_TFLOPS)
+    add("prefill: memory, head norm + gate", memory, lambda p: p._norm_gate(head_rows(p), rows(p), mixed_rows(p), dec.operand, T), nbytes=10.0 * T * MH * me)
+    add("prefill: memory, o + residual", memory, lambda p: p._out_rows(mixed_rows(p), p.k2, p.w_out, px, T), flops=2.0 * T * Hd * MH * me)
+    act_rows = dec.scratch.rows("act_rows", dense[0].ffp, T, dec.operand_torch)
+
+    def up_rows(p):
+        ck(L.dh_dense_matmul(p._normed_rows(px, T), dec.operand, p.kx, p.up.data_ptr(), p.kx, T, p.ff, p.kx, 1.0, None, None, None, 0, 0, act_rows, dec.operand,
+                             p.ffp, p.act))
+    add("prefill: dense ff, norm, up", dense, up_rows, flops=2.0 * T * Hd * ff)
+    add("prefill: dense ff, down + residual", dense, lambda p: p._out_rows(act_rows, p.ffp, p.down, px, T), flops=2.0 * T * Hd * ff)
+    me_ = experts[0].m
+    add("prefill: experts (norm, router, sort, products, sum)", experts, lambda p: p.rows(px, T, 0),
+        flops=6.0 * T * Hd * (me_["top"] * me_["ff"] + me_["shared"]["ff"]))
+    t.close()
+    return out
+
+
 def q4k_kernels(dec, s, T):
     from . import capi, synth
     L, ck, c = dec.L, capi.check, dec.cfg
@@ -182,30 +296,44 @@ def q4k_kernels(dec, s, T):
     return out
 
 
-def run(sizes, steps, warmup):
-    from . import decoder, dense_decoder
+def _measure(dec, prompt, steps, warmup, kernels, s):
+    pre, step = _throughput(dec, prompt, steps, warmup)
+    nbytes = dec.weight_bytes_per_token(PROMPT + steps // 2)
+    r = dict(prefill_tokens_per_s=round(pre, 1), decode_tokens_per_s=round(step, 1), decode_hbm_frac=round(nbytes * step / 1e9 / HBM_GBPS, 4))
+    if kernels in (zepavik_kernels, gusolorn_kernels):
+        dec.prefill(prompt, chunk=PROMPT)
+        r["replayed_tokens_per_s"] = round(_replayed(dec, PROMPT, steps), 1)
+    r["kernels"] = kernels(dec, s, PROMPT)
+    return r
+
+
+def run(design, sizes, steps, warmup):
+    from . import decoder, dense_decoder, gusolorn
     results = {}
     for name in sizes:
         s = SIZES[name]
         max_seq = PROMPT + warmup + steps + 80
         prompt = np.random.Generator(np.random.PCG64(1)).integers(0, VOCAB, PROMPT)
         r = dict(s, vocab=VOCAB, window=WINDOW, prompt=PROMPT)
-        cfg = zepavik_config(s, max_seq)
-        dec = dense_decoder.DenseDecoder(cfg, dense_decoder.random_weights(cfg, seed=2), max_seq)
-        pre, step = _throughput(dec, prompt, steps, warmup)
-        nbytes = dec.weight_bytes_per_token(PROMPT + steps // 2)
-        r["zepavik"] = dict(prefill_tokens_per_s=round(pre, 1), decode_tokens_per_s=round(step, 1),
-                            decode_hbm_frac=round(nbytes * step / 1e9 / HBM_GBPS, 4), kernels=zepavik_kernels(dec, s, PROMPT))
-        log("[bench] zepavik %s: prefill %.0f tok/s, decode %.1f tok/s" % (name, pre, step))
-        del dec
-        cfg = q4k_config(s, max_seq)
-        layers, embed, final_norm, cos, sin = decoder.random_model(cfg, seed=3, max_seq=max_seq)
-        dec = decoder.HipDecoder(cfg, layers, embed, final_norm, cos, sin, max_seq)
-        pre, step = _throughput(dec, prompt, steps, warmup)
-        nbytes = dec.weight_bytes_per_token(PROMPT + steps // 2)
-        r["q4k"] = dict(prefill_tokens_per_s=round(pre, 1), decode_tokens_per_s=round(step, 1),
-                        decode_hbm_frac=round(nbytes * step / 1e9 / HBM_GBPS, 4), kernels=q4k_kernels(dec, s, PROMPT))
-        log("[bench] q4k %s: prefill %.0f tok/s, decode %.1f tok/s" % (name, pre, step))
-        del dec
+        if design == "gusolorn":
+            r.update(MIXED[name])
+
+        def build(kind):
+            log("[bench] %s %s" % (kind, name))
+            if kind == "q4k":
+                cfg = q4k_config(s, max_seq)
+                layers, embed, final_norm, cos, sin = decoder.random_model(cfg, seed=3, max_seq=max_seq)
+                return decoder.HipDecoder(cfg, layers, embed, final_norm, cos, sin, max_seq)
+            if kind == "gusolorn":
+                cfg = gusolorn_config(s, MIXED[name])
+                return dense_decoder.DenseDecoder(cfg, gusolorn.random_weights(cfg, seed=4), max_seq)
+            cfg = zepavik_config(s, max_seq)
+            return dense_decoder.DenseDecoder(cfg, dense_decoder.random_weights(cfg, seed=2), max_seq)
+        kernels = dict(zepavik=zepavik_kernels, q4k=q4k_kernels, gusolorn=gusolorn_kernels)
+        for kind in (design, {"zepavik": "q4k", "gusolorn": "zepavik"}[design]):
+            dec = build(kind)
+            r[kind] = _measure(dec, prompt, steps, warmup, kernels[kind], s)
+            log("[bench] %s %s: prefill %.0f tok/s, decode %.1f tok/s" % (kind, name, r[kind]["prefill_tokens_per_s"], r[kind]["decode_tokens_per_s"]))
+            del dec
         results[name] = r
     return results

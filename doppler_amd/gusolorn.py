@@ -208,6 +208,11 @@ def random_weights(cfg, seed=0):
         if isinstance(entry, list):
             return np.stack([one(key, e) for e in entry])
         _, shape, kept = entry
+        if kept == "bits" and int(np.prod(shape)) >= 1 << 20:
+            # large matrices from random bits: sign and mantissa of +-[1, 2) times the power of two that gives about the same spread
+            r = g.integers(0, 256, shape, dtype=np.uint8).astype(np.uint16)
+            e = 127 if key == "embed" else 127 + int(np.round(np.log2(shape[-1] ** -0.5 / 1.53)))
+            return ((r & 0x80) << 8) | np.uint16(e << 7) | (r & 0x7F)
         z = g.standard_normal(shape, dtype=np.float32)
         if kept == "bits":
             return f32_to_bf16(z if key == "embed" else z * np.float32(shape[-1] ** -0.5))

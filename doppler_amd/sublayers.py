@@ -21,7 +21,7 @@ from .decoder import _dev_bytes
 
 ACTIVATIONS = {"relu2": capi.ACT_RELU2, "silu": capi.ACT_SILU, "gelu_tanh": capi.ACT_GELU, "gelu_erf": capi.ACT_GELU_ERF,
                None: capi.ACT_NONE}
-GEMV_MAX_K = 32768
+GEMV_MAX_K, GEMV_MAX_HEADS = 32768, 256
 
 
 def _up(n, m):
@@ -219,9 +219,18 @@ class MatrixMemory(_Sublayer):
 
     def step(self, pos, kv_len):
         d, f = self.dec, torch.float32
-        row, o, mixed = d.scratch.rows("row", self.n_in, 1, f), d.scratch.rows("heads", self.o_width, 1, f), d.scratch.rows("mixed", self.k2, 1, f)
+        row, o = d.scratch.rows("row", self.n_in, 1, f), d.scratch.rows("heads", self.o_width, 1, f)
         self._gemv(d.x.data_ptr(), True, self.w_in, self.n_in, self.kx, bias=self.bias.data_ptr(), out=row)
         capi.check(d.L.dh_mlstm_step(self.ref, row, self.memory.data_ptr(), o, pos, kv_len))
+        self._out_step(o, row)
+
+    def _out_step(self, o, row):
+        d, m = self.dec, self.m
+        if m["heads"] <= GEMV_MAX_HEADS:
+            capi.check(d.L.dh_dense_gemv_heads(o, row + 4 * self.g_off, self.head_norm.data_ptr(), m["heads"], self.VP, m["vdim"], self.eps,
+                                               self.w_out.data_ptr(), self.k2, self.hidden, self.k2, self.ls_ptr, d.x.data_ptr(), d.x.data_ptr()))
+            return
+        mixed = d.scratch.rows("mixed", self.k2, 1, torch.float32)
         self._norm_gate(o, row, mixed, capi.F32, 1)
         self._gemv(mixed, False, self.w_out, self.hidden, self.k2, residual=True)
 
