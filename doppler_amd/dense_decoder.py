@@ -151,6 +151,11 @@ class DenseDecoder(DecoderBase):
             self._rotary[base, dims] = tuple(_dev_bytes(t) for t in rotary_tables(base, dims, self.max_seq))
         return self._rotary[base, dims]
 
+    def capture_step(self, pos, want_logits=False, device_kv_len=True):
+        if not device_kv_len:
+            raise ValueError("captured steps of dense models read the key count on the device")
+        return super().capture_step(pos, want_logits)
+
     def _mixed_shapes(self):
         return {self._mixed_key(d["geo"]) for d in self._parallel()}
 

@@ -95,7 +95,7 @@ def tensors(cfg, seed, gain=2.0):
         E, ff = mlp["router"]["experts"], mlp["expert"]["ff"]
         t[p + "norm2"][:LEVELS] = 0.0
         t[p + "mlp.router"] = n(E, W, std=0.005)
-        t[p + "mlp.router"][np.arange(E), np.arange(E)] = 0.7
+        t[p + "mlp.router"][np.arange(E), np.arange(E)] = 0.703125
         parts = [("e%d" % k, ff) for k in range(E)]
         if mlp.get("shared"):
             parts.append(("shared", mlp["shared"]["ff"]))
