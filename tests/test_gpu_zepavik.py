@@ -374,7 +374,7 @@ def test_bad_specs_are_refused(L):
         setattr(spec, field, value)
         assert L.dh_attn_spec_kv_write(ctypes.byref(spec), rows.data_ptr(), a.kc.data_ptr(), a.vc.data_ptr(), 2, 0) != 0
         assert message in L.dh_last_error().decode(), (field, L.dh_last_error())
-    assert L.dh_dense_matmul(rows.data_ptr(), capi.F16, 64, rows.data_ptr(), 64, 1, 8, 64, 1.0, None, None, rows.data_ptr(), 8, 8, None, 0, 0, -1) != 0
+    assert L.dh_dense_matmul(rows.data_ptr(), 7, 64, rows.data_ptr(), 64, 1, 8, 64, 1.0, None, None, rows.data_ptr(), 8, 8, None, 0, 0, -1) != 0
     assert L.dh_dense_gemv(rows.data_ptr(), None, 0, 0.0, rows.data_ptr(), 100, 8, 100, 1.0, None, None, rows.data_ptr(), 8, None, -1) != 0
 
 
