@@ -77,29 +77,48 @@ __global__ __launch_bounds__(64 * WAVES) void gemv_kernel(const GemvArgs a) {
 
   // ---- the activation row
   if constexpr (HEADS) {
+    // weighted and gated on the way in; the squares are summed by eight lanes (whole heads: their sizes are multiples of 32), then by
+    // head, and the row in LDS is scaled last: one trip to memory
     __shared__ float inv_s[kMaxHeads];
-    const int hp = a.head_padded >> 2;                    // 16-byte pieces of a head
-    for (int h = wave; h < a.heads; h += WAVES) {
-      const float4* xh = reinterpret_cast<const float4*>(a.x) + (int64_t)h * hp;
-      float ss = 0.f;
-      for (int i = lane; i < hp; i += 64) {
-        const float4 v = xh[i];
-        ss = fmaf(v.x, v.x, ss); ss = fmaf(v.y, v.y, ss); ss = fmaf(v.z, v.z, ss); ss = fmaf(v.w, v.w, ss);
+    __shared__ float squares[kMaxK / 32];
+    const int hp = a.head_padded >> 2, live = a.heads * hp;       // 16-byte pieces of a head, of all heads
+    constexpr int BATCH = 4;                              // pieces requested at once
+    for (int i0 = tid; i0 < (a.K >> 2); i0 += THREADS * BATCH) {
+      float4 v[BATCH], w[BATCH], g[BATCH];
+#pragma unroll
+      for (int b = 0; b < BATCH; b++) {
+        const int i = i0 + THREADS * b;
+        v[b] = w[b] = g[b] = make_float4(0.f, 0.f, 0.f, 0.f);
+        if (i < live) {
+          v[b] = reinterpret_cast<const float4*>(a.x)[i];
+          w[b] = reinterpret_cast<const float4*>(a.norm_weight)[i];
+          g[b] = reinterpret_cast<const float4*>(a.gate)[i];
+        }
       }
-      ss = dh::wave_sum_uniform(ss);
-      if (lane == 0) inv_s[h] = 1.0f / sqrtf(ss / (float)a.head_size + a.eps);
+#pragma unroll
+      for (int b = 0; b < BATCH; b++) {
+        const int i = i0 + THREADS * b;
+        if (i >= (a.K >> 2)) break;                       // sixteen lanes at a time: K is a multiple of 64
+        float4 y = v[b];
+        float ss = fmaf(y.x, y.x, fmaf(y.y, y.y, fmaf(y.z, y.z, y.w * y.w)));
+        y.x = y.x * w[b].x * __frcp_rn(1.0f + __expf(-g[b].x)); y.y = y.y * w[b].y * __frcp_rn(1.0f + __expf(-g[b].y));
+        y.z = y.z * w[b].z * __frcp_rn(1.0f + __expf(-g[b].z)); y.w = y.w * w[b].w * __frcp_rn(1.0f + __expf(-g[b].w));
+        planes[(i & 1) * np + (i >> 1)] = y;
+        ss = dh::group_combine<1, 8>(ss, dh::AddOp());
+        if ((i & 7) == 0) squares[i >> 3] = ss;
+      }
     }
     __syncthreads();
-    for (int i = tid; i < (a.K >> 2); i += THREADS) {
-      float4 v = make_float4(0.f, 0.f, 0.f, 0.f);
-      if (i < a.heads * hp) {
-        v = reinterpret_cast<const float4*>(a.x)[i];
-        const float4 w = reinterpret_cast<const float4*>(a.norm_weight)[i], g = reinterpret_cast<const float4*>(a.gate)[i];
-        const float f = inv_s[i / hp];
-        v.x = v.x * f * w.x / (1.0f + expf(-g.x)); v.y = v.y * f * w.y / (1.0f + expf(-g.y));
-        v.z = v.z * f * w.z / (1.0f + expf(-g.z)); v.w = v.w * f * w.w / (1.0f + expf(-g.w));
-      }
-      planes[(i & 1) * np + (i >> 1)] = v;
+    for (int h = tid; h < a.heads; h += THREADS) {
+      float ss = 0.f;
+      for (int k = h * (hp >> 3); k < (h + 1) * (hp >> 3); k++) ss += squares[k];
+      inv_s[h] = 1.0f / sqrtf(ss / (float)a.head_size + a.eps);
+    }
+    __syncthreads();
+    for (int i = tid; i < live; i += THREADS) {
+      const float f = inv_s[i / hp];
+      float4& v = planes[(i & 1) * np + (i >> 1)];
+      v.x *= f; v.y *= f; v.z *= f; v.w *= f;
     }
   } else {
     const float4* xg = reinterpret_cast<const float4*>(a.x);
@@ -213,6 +232,13 @@ int dispatch(const char* op, const GemvArgs& a, int* parts) {
   // workgroups that are resident at once share the activation row's preparation as widely as the LDS allows
   const int cus = dh::num_cus();
   static const int env_r = dh::tuning_int("DH_DENSE_GEMV_R", 0);
+  if constexpr (HEADS) {
+    // every workgroup reads three rows to prepare one: wide workgroups, as long as there is one for every compute unit
+    static const int env_w = dh::tuning_int("DH_GEMV_HEADS_WAVES", 0);
+    const int waves = env_w ? env_w : a.N >= 16 * cus ? 16 : a.N >= 8 * cus ? 8 : 4;
+    if (a.K <= 8192 && waves == 16) return launch<1, 8, 16, ARGMAX, HEADS>(op, a, cus, parts);
+    if (a.K <= 8192 && waves == 8) return launch<1, 8, 8, ARGMAX, HEADS>(op, a, 2 * cus, parts);
+  }
   const bool two = env_r ? env_r == 2 : a.K <= 4096 && (int64_t)a.N >= (int64_t)64 * cus;
   if (a.K <= 8192) {
     const int max_grid = ARGMAX ? std::min(4 * cus, dh::kMaxParts) : 4 * cus;
@@ -273,8 +299,8 @@ int dh_dense_gemv_heads(const float* d_x, const float* d_gate, const float* d_we
   const char* op = "dh_dense_gemv_heads";
   DH_REQUIRE_INIT(op);
   if (int rc = check(op, d_x, nullptr, 0, eps, d_W, ldw, N, K)) return rc;
-  if (H <= 0 || H > kMaxHeads || size <= 0 || padded < size || padded % 4 || (int64_t)H * padded > K)
-    return dh::fail(1, "[%s] %d heads (at most %d) of %d elements, %d apart, in a row of %d", op, H, kMaxHeads, size, padded, K);
+  if (H <= 0 || H > kMaxHeads || size <= 0 || padded < size || padded % 32 || (int64_t)H * padded > K)
+    return dh::fail(1, "[%s] %d heads (at most %d) of %d elements, %d apart (a multiple of 32), in a row of %d", op, H, kMaxHeads, size, padded, K);
   if (!d_gate || !d_weight || !d_C) return dh::fail(1, "[%s] null pointer", op);
   if ((reinterpret_cast<uintptr_t>(d_gate) | reinterpret_cast<uintptr_t>(d_weight)) & 15) return dh::fail(1, "[%s] gate and weight must be 16-byte aligned", op);
   if (d_x == d_C) return dh::fail(1, "[%s] the output must not be the activation row", op);

@@ -384,7 +384,7 @@ int dh_dense_gemv_scaled(const float* d_x, const float* d_norm_weight, int hidde
                          int K, float alpha, const float* d_bias, const float* d_col_scale, const float* d_residual, float* d_C,
                          int n_first, float* d_C2, int activation);
 /* C = (W y) * col_scale + residual with y the gated, normed heads of dh_head_norm_gate: x_h / rms(x_h) * weight * sigmoid(gate); at most
- * 256 heads of `padded` floats, K >= H * padded. */
+ * 256 heads of `padded` floats (a multiple of 32), K >= H * padded. */
 int dh_dense_gemv_heads(const float* d_x, const float* d_gate, const float* d_weight, int H, int padded, int size, float eps, const void* d_W,
                         int ldw, int N, int K, const float* d_col_scale, const float* d_residual, float* d_C);
 /* dh_lmhead_argmax_f16_rmsnorm for an untied bf16 head: logits = alpha * W norm(x), token = their argmax (ties to
