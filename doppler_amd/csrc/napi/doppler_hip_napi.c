@@ -456,6 +456,80 @@ FN(js_attn_spec_decode) {
   return ret_rc(env, dh_attn_spec_decode(s, (const float*)qkv, ck, cv, (float*)out, pos, (const uint32_t*)kvLen, maxKvLen, ws));
 }
 
+/* ---- sequential layers; their specs travel as bytes too ---- */
+FN(js_sublayer_struct_bytes) {
+  (void)info;
+  napi_value arr;
+  const size_t sizes[3] = {sizeof(dh_latent), sizeof(dh_mlstm), sizeof(dh_experts)};
+  napi_create_array_with_length(env, 3, &arr);
+  for (uint32_t i = 0; i < 3; i++) napi_set_element(env, arr, i, ret_num(env, (double)sizes[i]));
+  return arr;
+}
+static const void* arg_struct(napi_env env, napi_value v, size_t size) {
+  void* data = NULL; size_t len = 0;
+  if (!arg_bytes(env, v, &data, &len)) return NULL;
+  if (len < size) {
+    napi_throw_error(env, NULL, "doppler_hip: the spec bytes are shorter than the struct");
+    return NULL;
+  }
+  return data;
+}
+#define SPEC(type) const type* s = (const type*)arg_struct(env, a[0], sizeof(type)); if (!s) return NULL
+FN(js_dense_matmul_scaled) {
+  ARGS(19); P(0, A); I(1, adt); I(2, lda); P(3, W); I(4, ldw); I(5, M); I(6, N); I(7, K); F(8, alpha); P(9, bias); P(10, cs); P(11, res);
+  P(12, C); I(13, ldc); I(14, first); P(15, C2); I(16, c2dt); I(17, ldc2); I(18, act);
+  return ret_rc(env, dh_dense_matmul_scaled(A, adt, lda, W, ldw, M, N, K, alpha, (const float*)bias, (const float*)cs, (const float*)res,
+                                            (float*)C, ldc, first, C2, c2dt, ldc2, act));
+}
+FN(js_dense_gemv_scaled) {
+  ARGS(16); P(0, x); P(1, nw); I(2, hid); F(3, eps); P(4, W); I(5, ldw); I(6, N); I(7, K); F(8, alpha); P(9, bias); P(10, cs); P(11, res);
+  P(12, C); I(13, first); P(14, C2); I(15, act);
+  return ret_rc(env, dh_dense_gemv_scaled((const float*)x, (const float*)nw, hid, eps, W, ldw, N, K, alpha, (const float*)bias,
+                                          (const float*)cs, (const float*)res, (float*)C, first, (float*)C2, act));
+}
+FN(js_dense_gemv_heads) {
+  ARGS(14); P(0, x); P(1, g); P(2, w); I(3, H); I(4, padded); I(5, size); F(6, eps); P(7, W); I(8, ldw); I(9, N); I(10, K); P(11, cs);
+  P(12, res); P(13, C);
+  return ret_rc(env, dh_dense_gemv_heads((const float*)x, (const float*)g, (const float*)w, H, padded, size, eps, W, ldw, N, K,
+                                         (const float*)cs, (const float*)res, (float*)C));
+}
+FN(js_head_norm_gate) {
+  ARGS(13); P(0, x); I(1, ldx); P(2, g); I(3, ldg); P(4, w); P(5, out); I(6, dt); I(7, ldo); I(8, rows); I(9, H); I(10, padded); I(11, size);
+  F(12, eps);
+  return ret_rc(env, dh_head_norm_gate((const float*)x, ldx, (const float*)g, ldg, (const float*)w, out, dt, ldo, rows, H, padded, size, eps));
+}
+FN(js_latent_rows) {
+  ARGS(5); P(1, rows); P(2, cache); I(3, T); I(4, start); SPEC(dh_latent);
+  return ret_rc(env, dh_latent_rows(s, (float*)rows, cache, T, start));
+}
+FN(js_latent_prefill_workspace_bytes) { ARGS(3); I(1, T); I(2, start); SPEC(dh_latent); return ret_num(env, (double)dh_latent_prefill_workspace_bytes(s, T, start)); }
+FN(js_latent_prefill) {
+  ARGS(9); P(1, rows); P(2, cache); P(3, ws); P(4, out); I(5, dt); I(6, ld); I(7, T); I(8, start); SPEC(dh_latent);
+  return ret_rc(env, dh_latent_prefill(s, (const float*)rows, cache, ws, out, dt, ld, T, start));
+}
+FN(js_latent_decode_workspace_bytes) { ARGS(2); I(1, kv); SPEC(dh_latent); return ret_num(env, (double)dh_latent_decode_workspace_bytes(s, kv)); }
+FN(js_latent_decode) {
+  ARGS(8); P(1, row); P(2, cache); P(3, out); I(4, pos); P(5, kvLen); I(6, maxKvLen); P(7, ws); SPEC(dh_latent);
+  return ret_rc(env, dh_latent_decode(s, (const float*)row, cache, (float*)out, pos, (const uint32_t*)kvLen, maxKvLen, ws));
+}
+FN(js_mlstm_state_bytes) { ARGS(1); SPEC(dh_mlstm); return ret_num(env, (double)dh_mlstm_state_bytes(s)); }
+FN(js_mlstm_step) {
+  ARGS(6); P(1, row); P(2, state); P(3, out); I(4, pos); P(5, kvLen); SPEC(dh_mlstm);
+  return ret_rc(env, dh_mlstm_step(s, (const float*)row, state, (float*)out, pos, (const uint32_t*)kvLen));
+}
+FN(js_mlstm_prefill_workspace_bytes) { ARGS(2); I(1, T); SPEC(dh_mlstm); return ret_num(env, (double)dh_mlstm_prefill_workspace_bytes(s, T)); }
+FN(js_mlstm_prefill) {
+  ARGS(8); P(1, rows); P(2, state); P(3, ws); P(4, out); I(5, ld); I(6, T); I(7, start); SPEC(dh_mlstm);
+  return ret_rc(env, dh_mlstm_prefill(s, (const float*)rows, state, ws, (float*)out, ld, T, start));
+}
+FN(js_experts_step_workspace_bytes) { ARGS(1); SPEC(dh_experts); return ret_num(env, (double)dh_experts_step_workspace_bytes(s)); }
+FN(js_experts_step) { ARGS(3); P(1, x); P(2, ws); SPEC(dh_experts); return ret_rc(env, dh_experts_step(s, (float*)x, ws)); }
+FN(js_experts_prefill_workspace_bytes) { ARGS(3); I(1, dt); I(2, T); SPEC(dh_experts); return ret_num(env, (double)dh_experts_prefill_workspace_bytes(s, dt, T)); }
+FN(js_experts_prefill) {
+  ARGS(7); P(1, h); I(2, dt); P(3, x); I(4, ldx); P(5, ws); I(6, T); SPEC(dh_experts);
+  return ret_rc(env, dh_experts_prefill(s, h, dt, (float*)x, ldx, ws, T));
+}
+
 static napi_value module_init(napi_env env, napi_value exports) {
   static const struct { const char* name; napi_callback fn; } table[] = {
       {"graphBegin", js_graph_begin}, {"graphEnd", js_graph_end}, {"graphLaunch", js_graph_launch}, {"graphSetMaxPosition", js_graph_set_max_position}, {"graphPrepare", js_graph_prepare},
@@ -490,6 +564,14 @@ static napi_value module_init(napi_env env, napi_value exports) {
       {"embedSum", js_embed_sum}, {"rmsnormRows", js_rmsnorm_rows}, {"attnSpecBytes", js_attn_spec_bytes},
       {"attnSpecWorkspaceBytes", js_attn_spec_workspace_bytes}, {"attnSpecKvWrite", js_attn_spec_kv_write},
       {"attnSpecPrefill", js_attn_spec_prefill}, {"attnSpecDecode", js_attn_spec_decode},
+      {"sublayerStructBytes", js_sublayer_struct_bytes}, {"denseMatmulScaled", js_dense_matmul_scaled},
+      {"denseGemvScaled", js_dense_gemv_scaled}, {"denseGemvHeads", js_dense_gemv_heads}, {"headNormGate", js_head_norm_gate},
+      {"latentRows", js_latent_rows}, {"latentPrefillWorkspaceBytes", js_latent_prefill_workspace_bytes}, {"latentPrefill", js_latent_prefill},
+      {"latentDecodeWorkspaceBytes", js_latent_decode_workspace_bytes}, {"latentDecode", js_latent_decode},
+      {"mlstmStateBytes", js_mlstm_state_bytes}, {"mlstmStep", js_mlstm_step},
+      {"mlstmPrefillWorkspaceBytes", js_mlstm_prefill_workspace_bytes}, {"mlstmPrefill", js_mlstm_prefill},
+      {"expertsStepWorkspaceBytes", js_experts_step_workspace_bytes}, {"expertsStep", js_experts_step},
+      {"expertsPrefillWorkspaceBytes", js_experts_prefill_workspace_bytes}, {"expertsPrefill", js_experts_prefill},
   };
   for (size_t i = 0; i < sizeof(table) / sizeof(table[0]); i++) {
     napi_value fn;

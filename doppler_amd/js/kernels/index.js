@@ -13,6 +13,10 @@ export {
   recordEmbedSum, recordRMSNormRows, recordDenseMatmul, recordDenseGemv, recordDenseLmHeadArgmax, packAttnSpec,
   recordAttnSpecKVWrite, recordAttnSpecPrefill, recordAttnSpecDecode,
 } from './dense.js';
+export {
+  packLatent, packMlstm, packExperts, recordDenseMatmulScaled, recordDenseGemvScaled, recordDenseGemvHeads, recordHeadNormGate, recordLatentRows,
+  recordLatentPrefill, recordLatentDecode, recordMlstmStep, recordMlstmPrefill, recordExpertsStep, recordExpertsPrefill,
+} from './sublayers.js';
 export { runRMSNorm, recordRMSNorm } from './rmsnorm.js';
 export { runRMSNormQK, recordRMSNormQK, canUseRMSNormQK } from './rmsnorm-qk.js';
 export {

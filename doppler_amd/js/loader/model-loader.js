@@ -4,16 +4,16 @@ import fs from 'fs';
 import path from 'path';
 
 import { loadDecoderWeights } from './rdrr-loader.js';
+import { loadGusolorn } from './gusolorn-loader.js';
 import { loadZepavik } from './zepavik-loader.js';
 import { HipTextDecoder } from '../pipeline/decode-step.js';
 import { DenseTextDecoder } from '../pipeline/dense-decoder.js';
 
-const ARCHITECTURES = {
-  Zepavik: (dir, options) => {
-    const { config, weights } = loadZepavik(dir, options.maxSeq);
-    return new DenseTextDecoder(Object.assign({ compute: options.dtype === 'float32' ? 'f32' : 'bf16' }, config, options.config), weights);
-  },
+const dense = (load) => (dir, options) => {
+  const { config, weights } = load(dir, options.maxSeq);
+  return new DenseTextDecoder(Object.assign({ compute: options.dtype === 'float32' ? 'f32' : 'bf16' }, config, options.config), weights);
 };
+const ARCHITECTURES = { Zepavik: dense(loadZepavik), Gusolorn: dense(loadGusolorn) };
 
 // options: {maxSeq, dtype: 'bfloat16'|'float32', config: extra decoder settings}
 export function loadModel(dir, options = {}) {

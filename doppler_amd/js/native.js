@@ -20,7 +20,7 @@ try {
 export const DTYPE = Object.freeze({ f32: 0, f16: 1, bf16: 2 });
 export const ACT = Object.freeze({ silu: 0, gelu: 1 });
 // plain activations of the dense products
-export const DENSE_ACT = Object.freeze({ silu: 0, gelu_tanh: 1, relu2: 2, none: -1 });
+export const DENSE_ACT = Object.freeze({ silu: 0, gelu_tanh: 1, relu2: 2, gelu_erf: 3, none: -1 });
 export const KV_LAYOUT = Object.freeze({ contiguous: 0, ring: 1 });
 
 let initialised = false;

@@ -1,4 +1,4 @@
-// Decoder with dense bf16 weights: the JavaScript side of doppler_amd/dense_decoder.py.  A parallel layer
+// Decoder with dense bf16 weights: the JavaScript side of doppler_amd/dense_decoder.py.  Layers are sequential (sublayers.js) or parallel:
 //   x <- x + mixer(norm(x)) + ff(norm(x))
 // is two products: [q | k | v | gate | up] = W_in norm(x), and x += W_out [attention | act(up)].  Head sizes are padded
 // to multiples of 8 and every k extent to a multiple of 64 with zeros.
@@ -7,6 +7,7 @@ import {
   recordDenseLmHeadArgmax, packAttnSpec, recordAttnSpecKVWrite, recordAttnSpecPrefill, recordAttnSpecDecode, recordCheckFiniteness,
 } from '../kernel-selector.js';
 import { getNative } from '../native.js';
+import { SequentialLayer } from './sublayers.js';
 import { TextDecoder, bufferWindow, upload } from './text-decoder.js';
 
 const GEMV_MAX_K = 32768;
@@ -45,9 +46,10 @@ function stackLayer(mixer, mlp, w, hidden) {
 
 export class DenseTextDecoder extends TextDecoder {
   // config: {hidden, vocab, eps, logitScale, maxPositions, maxSeq, compute: 'bf16'|'f32', bigram: {buckets, mulPrev, mulCur}|null,
-  //          layers: [{mixer: {heads, kvHeads, dim, vdim, window, scale, logBias, valueNorm, gate}, mlp: {ff, activation}|null}]}
+  //          layers: [{mixer: {heads, kvHeads, dim, vdim, window, scale, logBias, valueNorm, gate}, mlp: {ff, activation}|null}, or
+  //                   {sequential: true, mixer: {type, ..}, mlp: {type, ..}|null}]}
   // weights: {embed, bigram, pos, head (Uint16Array bf16 bits), finalNorm, layers: [{norm, qBias, kBias, vBias, biasR1, biasR2
-  //           (Float32Array), q, k, v, gate, o, up, down (Uint16Array)}]}
+  //           (Float32Array), q, k, v, gate, o, up, down (Uint16Array)}, or what SequentialLayer takes]}
   constructor(config, weights) {
     super(config);
     const c = config;
@@ -59,7 +61,13 @@ export class DenseTextDecoder extends TextDecoder {
     const padded = (v) => { const out = new Float32Array(this.kx); out.set(v); return upload(out, 'norm'); };
     let workspace = 256, qkv = 1;
     this.mixed = new Map();
+    this.scratchBuffers = new Map();
+    this.rotaryTables = new Map();
+    this.operandBytes = this.operand === 'bf16' ? 2 : 4;
+    const earlier = [];
+    const keep = (layer) => { earlier.push(layer); return layer; };
     this.layers = weights.layers.map((w, i) => {
+      if (c.layers[i].sequential) return keep({ sublayers: new SequentialLayer(this, c.layers[i], w, earlier.map((l) => l.sublayers)) });
       const m = c.layers[i].mixer, mlp = c.layers[i].mlp;
       const { g, wIn, bias, wOut } = stackLayer(m, mlp, w, c.hidden);
       if (g.k2 > GEMV_MAX_K) throw new Error(`[DenseTextDecoder] layer ${i}: rows of ${g.k2} are not served by this host`);
@@ -78,7 +86,7 @@ export class DenseTextDecoder extends TextDecoder {
       qkv = Math.max(qkv, g.nFirst);
       const key = `${g.attnCols + g.ff}/${g.k2}`;
       if (!this.mixed.has(key)) this.mixed.set(key, this.zeroed(g.k2 * 4, 'mixed'));
-      return { buffers: l, g, spec, key, activation: mlp ? mlp.activation : 'none' };
+      return keep({ buffers: l, g, spec, key, activation: mlp ? mlp.activation : 'none' });
     });
     this.tables = {
       embed: upload(weights.embed, 'embed'), bigram: c.bigram ? upload(weights.bigram, 'bigram') : null,
@@ -97,6 +105,30 @@ export class DenseTextDecoder extends TextDecoder {
     const b = acquireBuffer(up(bytes, 4), undefined, label);
     getNative().fillZero(b.ptr, 0, up(bytes, 4));
     return b;
+  }
+
+  // A buffer all layers share, by name and row width (what lies behind a row's elements stays zero), grown to the most rows asked for.
+  scratch(name, width, count, elementBytes) {
+    const key = `${name}/${width}/${elementBytes}`, bytes = width * count * elementBytes;
+    const held = this.scratchBuffers.get(key);
+    if (held && held.size >= bytes) return held;
+    if (held) releaseBuffer(held);
+    const buffer = this.zeroed(bytes, name);
+    this.scratchBuffers.set(key, buffer);
+    return buffer;
+  }
+
+  rotary(base, dims, make) {
+    const key = `${base}/${dims}`;
+    if (!this.rotaryTables.has(key)) {
+      const t = make(base, dims, this.config.maxSeq);
+      this.rotaryTables.set(key, { cos: upload(t.cos, 'cos'), sin: upload(t.sin, 'sin') });
+    }
+    return this.rotaryTables.get(key);
+  }
+
+  carriesState() {
+    return this.layers.some((l) => l.sublayers && l.sublayers.recurrent);
   }
 
   deviceKvLenServed() {
@@ -120,19 +152,24 @@ export class DenseTextDecoder extends TextDecoder {
     const c = this.config, s = this.step;
     const kvLen = options.deviceKvLen ? bufferWindow(this.ids, 4, 4) : null;
     for (let li = 0; li < this.layers.length; li++) {
-      const { buffers: l, g, spec, key, activation } = this.layers[li];
-      const mixed = this.mixed.get(key);
-      recordDenseGemv(recorder, {
-        input: s.x, normWeight: l.norm, hidden: c.hidden, eps: c.eps, weight: l.wIn, ldw: g.kx, N: g.n, K: g.kx, bias: l.bias, output: s.qkv,
-        nFirst: g.nFirst, output2: g.ff ? bufferWindow(mixed, 4 * g.attnCols, 4 * g.ff) : null, activation,
-      });
-      recordAttnSpecDecode(recorder, spec, s.qkv, l.cacheK, l.cacheV, mixed, pos, kvLen, c.maxSeq, s.attn);
-      recordDenseGemv(recorder, { input: mixed, weight: l.wOut, ldw: g.k2, N: c.hidden, K: g.k2, residual: s.x, output: s.x, nFirst: c.hidden });
+      const layer = this.layers[li];
+      if (layer.sublayers) layer.sublayers.step(recorder, pos, kvLen);
+      else this.recordParallelLayer(recorder, layer, pos, kvLen);
       if (this.finitenessGuard) {
         recordCheckFiniteness(recorder, x, c.hidden, this.finitenessStatus, li, pos, this.finitenessAbsThreshold);
       }
     }
     return x;
+  }
+
+  recordParallelLayer(recorder, { buffers: l, g, spec, key, activation }, pos, kvLen) {
+    const c = this.config, s = this.step, mixed = this.mixed.get(key);
+    recordDenseGemv(recorder, {
+      input: s.x, normWeight: l.norm, hidden: c.hidden, eps: c.eps, weight: l.wIn, ldw: g.kx, N: g.n, K: g.kx, bias: l.bias, output: s.qkv,
+      nFirst: g.nFirst, output2: g.ff ? bufferWindow(mixed, 4 * g.attnCols, 4 * g.ff) : null, activation,
+    });
+    recordAttnSpecDecode(recorder, spec, s.qkv, l.cacheK, l.cacheV, mixed, pos, kvLen, c.maxSeq, s.attn);
+    recordDenseGemv(recorder, { input: mixed, weight: l.wOut, ldw: g.k2, N: c.hidden, K: g.k2, residual: s.x, output: s.x, nFirst: c.hidden });
   }
 
   async recordNormedLmHead(recorder, temps, row, tokenOut, tokenIndex, logitsOutput) {
@@ -148,7 +185,7 @@ export class DenseTextDecoder extends TextDecoder {
     if (!this.batch || this.batch.rows < T) {
       this.releaseBatch();
       const mixed = new Map();
-      for (const { g, key } of this.layers) {
+      for (const { g, key } of this.layers.filter((l) => !l.sublayers)) {
         if (!mixed.has(key)) mixed.set(key, this.zeroed(T * g.k2 * elem, 'prefill_mixed'));
       }
       this.batch = {
@@ -158,7 +195,12 @@ export class DenseTextDecoder extends TextDecoder {
     }
     const b = this.batch;
     recordEmbedSum(recorder, this.embedding(ids, 1, ids, b.x, T, pos, null));
-    for (const { buffers: l, g, spec, key, activation } of this.layers) {
+    for (const layer of this.layers) {
+      if (layer.sublayers) {
+        layer.sublayers.rows(recorder, b.x, T, pos);
+        continue;
+      }
+      const { buffers: l, g, spec, key, activation } = layer;
       const mixed = b.mixed.get(key);
       recordRMSNormRows(recorder, {
         input: b.x, ldIn: this.kx, rows: null, weight: l.norm, output: b.normed, dtype: this.operand, ldOut: this.kx, count: T,
@@ -187,7 +229,8 @@ export class DenseTextDecoder extends TextDecoder {
 
   releaseWeights() {
     this.releaseBatch();
-    for (const l of this.layers) Object.keys(l.buffers).forEach((k) => releaseBuffer(l.buffers[k]));
-    for (const b of Array.from(this.mixed.values()).concat(Object.values(this.step), Object.values(this.tables))) releaseBuffer(b);
+    for (const l of this.layers) (l.sublayers ? l.sublayers.ownBuffers() : Object.values(l.buffers)).forEach(releaseBuffer);
+    const shared = [].concat(...Array.from(this.rotaryTables.values()).map((t) => [t.cos, t.sin]), Array.from(this.scratchBuffers.values()));
+    for (const b of Array.from(this.mixed.values()).concat(Object.values(this.step), Object.values(this.tables), shared)) releaseBuffer(b);
   }
 }

@@ -10,6 +10,8 @@
 //   recordPrefillChunk(recorder, temps, ids, part, pos)         a portion; returns its final residual rows
 //                                                               {buffer, rowFloats}; ids: device words [before, part...]
 //   deviceKvLenServed()                                         whether captured steps read the key count on the device
+//   carriesState()                                              whether its layers carry recurrent state: positions must then follow
+//                                                               one another, or start again at 0
 //   releaseWeights()
 import {
   createTensor, acquireBuffer, releaseBuffer, uploadData, readBufferSlice, createCommandRecorder, recordGPUSample,
@@ -60,6 +62,18 @@ export class TextDecoder {
     this.readback = null;
     // tokens fed so far by position: a model whose embedding reads the previous token finds it here
     this.history = new Uint32Array(config.maxSeq);
+    this.statePos = 0;     // the position recurrent state is ready for
+  }
+
+  carriesState() {
+    return false;
+  }
+
+  advance(pos, tokens) {
+    if (pos !== 0 && pos !== this.statePos && this.carriesState()) {
+      throw new Error(`the sequence's recurrent state stands at position ${this.statePos}, not at ${pos}`);
+    }
+    this.statePos = pos + tokens;
   }
 
   remember(pos, tokens) {
@@ -105,6 +119,7 @@ export class TextDecoder {
       const part = tokens.slice(c0, c0 + chunk);
       T = part.length;
       const pos = startPos + c0;
+      this.advance(pos, T);
       uploadData(ids, new Uint32Array([this.tokenBefore(pos)].concat(Array.from(part))));
       rows = await this.recordPrefillChunk(recorder, temps, ids, part, pos);
     }
@@ -142,6 +157,8 @@ export class TextDecoder {
       // the ops take no cache capacity: a position past the caches would write K/V out of bounds
       throw new Error(`[decodeStep] position ${pos} is outside the KV cache (maxSeq=${c.maxSeq})`);
     }
+    // a captured step (its key count on the device) is recorded here and runs when it is replayed
+    if (!options.deviceKvLen) this.advance(pos, 1);
     const tokenOut = options.tokenOutBuffer || this.tokenOut, tokenIndex = options.tokenOutIndex || 0;
     let x = await this.recordEmbedding(recorder, temps, options.idsBuffer || this.ids, options.prevBuffer || bufferWindow(this.ids, 8, 4),
       pos, options);
@@ -274,6 +291,7 @@ export class TextDecoder {
       throw new Error(`[decodeStepGraph] position ${pos} is outside the KV cache (maxSeq=${c.maxSeq})`);
     }
     if (!this.graph) return this.captureDecodeStep(token, pos);
+    this.advance(pos, 1);
     // token id and key count travel together; the attention kernels of the captured step read the count
     this.uploadStep(token, pos, pos + 1);
     getNative().graphLaunch(this.graph, pos);

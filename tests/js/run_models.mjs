@@ -1,4 +1,4 @@
-// Driver of tests/test_gpu_zepavik_js.py: node run_zepavik.mjs jobs.json -> one JSON line with the tokens of every job.
+// Driver of the tests of the JavaScript host with whole models: node run_models.mjs jobs.json -> one JSON line with the tokens of every job.
 import fs from 'fs';
 import { loadModel } from '../../doppler_amd/js/loader/model-loader.js';
 
@@ -31,6 +31,12 @@ async function main() {
       for (let i = 1; i < j.count; i++) {
         const pos = n + i - 1;
         tokens.push(i % 5 === 4 ? await dec.decodeStep(tokens[i - 1], pos) : await dec.decodeStepGraph(tokens[i - 1], pos));
+      }
+    } else if (j.mode === 'order') {
+      tokens = [];
+      await dec.prefill(j.prompt);
+      for (const run of [() => dec.decodeStep(1, n + 2), () => dec.prefill([1, 2], n - 1), () => dec.decodeStep(1, n)]) {
+        try { await run(); tokens.push('ran'); } catch (e) { tokens.push(e.message); }
       }
     } else if (j.mode === 'guard') {
       let message = 'did not throw';

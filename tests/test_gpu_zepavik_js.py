@@ -79,7 +79,7 @@ def test_js_host_generates_what_the_python_host_does(tmp_path):
         want[key] = ["FinitenessError: F16 bounds exceeded during generation (layer 1, step 40)"]
     path = str(tmp_path / "jobs.json")
     json.dump(jobs, open(path, "w"))
-    r = subprocess.run([NODE, os.path.join(ROOT, "tests", "js", "run_zepavik.mjs"), path], cwd=ROOT, capture_output=True, text=True, timeout=110)
+    r = subprocess.run([NODE, os.path.join(ROOT, "tests", "js", "run_models.mjs"), path], cwd=ROOT, capture_output=True, text=True, timeout=110)
     assert r.returncode == 0, r.stderr[-3000:]
     got = json.loads(r.stdout.strip().splitlines()[-1])
     for key in want:
