@@ -1,9 +1,10 @@
 """Throughput of a design beside the closest decoder the package serves, at sizes that resemble a real model's layers.
 
-Gusolorn (sequential layers: latent attention with a dense feed-forward, two of matrix memory with experts, and again) against Zepavik
-with the same width, heads, layer count, window and active feed-forward width.  Zepavik (dense bf16, parallel layers, windowed attention) against the Q4_K decoder with the same width, heads, feed-forward
-width and layer count: prefill and decode tokens/s, and per kernel the share of its roofline (8 TB/s of HBM, 2.5
-PFLOP/s on the matrix cores).  Random weights; kernels cycle through more weights than the caches hold.
+Gusolorn (sequential layers: latent attention with a dense feed-forward, two of matrix memory with experts, and again) against
+Zepavik with the same width, heads, layer count, window and active feed-forward width.  Zepavik (dense bf16, parallel layers, windowed
+attention) against the Q4_K decoder with the same width, heads, feed-forward width and layer count.  Prefill and decode tokens/s, and
+per kernel the share of its roofline (8 TB/s of HBM, 2.5 PFLOP/s on the matrix cores, 157 TFLOP/s for 32-bit products).  Random
+weights; kernels cycle through more weights than the caches hold.
 """
 import ctypes
 import sys
