@@ -326,7 +326,7 @@ def test_dense_feed_forward(L, tmp_path, ff, dtype):
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
-@pytest.mark.parametrize("E,top,ff,limit,shared", [(5, 2, 36, 0.8, (52, 1.3)), (8, 1, 64, 1.0, (128, 1.5)), (3, 3, 130, 0.2, None), (8, 7, 20, 5.0, (7, 0.1)),
+@pytest.mark.parametrize("E,top,ff,limit,shared", [(5, 2, 36, 0.8, (52, 1.3)), (8, 1, 72, 1.2, (136, 1.7)), (3, 3, 130, 0.2, None), (8, 7, 20, 5.0, (7, 0.1)),
                                                    (1, 1, 1, 1.0, None)])
 def test_experts(L, tmp_path, E, top, ff, limit, shared, dtype):
     n = 300
